@@ -1,25 +1,62 @@
-"""Model factory: named presets -> decoder instances.
+"""Model registry: preset names and checkpoint folders -> decoder instances.
 
 BASELINE.json configs name two decoder families: Llama-3-8B (config 3, the
-flagship agent LLM) and Mixtral-8x7B MoE (config 5).
+flagship agent LLM) and Mixtral-8x7B MoE (config 5); Luzalorn is a
+config-driven decoder of retention and latent-attention layers.
+
+`build_model(name)` takes a preset name (random weights) or a folder with
+config.json + model.safetensors; a folder's class is chosen by the
+'architecture' its config.json names (ARCHITECTURES).
 """
 
 from __future__ import annotations
+
+import json
+import os
+
+
+def _luzalorn():
+    from .luzalorn import LuzalornModel
+    return LuzalornModel
+
+
+# config.json 'architecture' -> loader of the model class
+ARCHITECTURES = {"Luzalorn": _luzalorn}
+
+
+def load_model(folder: str, device: str = "cuda", dtype=None, **kw):
+    """A model with the weights of `folder`."""
+    with open(os.path.join(folder, "config.json"), encoding="utf-8") as fh:
+        config = json.load(fh)
+    arch = config.get("architecture")
+    if arch not in ARCHITECTURES:
+        raise ValueError(f"{folder}: unknown architecture {arch!r} "
+                         f"(known: {', '.join(sorted(ARCHITECTURES))})")
+    return ARCHITECTURES[arch]().from_folder(
+        folder, config, device=device, dtype=dtype or _dtype(device), **kw)
+
+
+def _dtype(device):
+    import torch
+    return torch.bfloat16 if str(device).startswith("cuda") \
+        else torch.float32
 
 
 def build_model(name: str, device: str = "cuda", dtype=None, seed: int = 0,
                 tp_rank: int = 0, tp_size: int = 1, tp_group=None,
                 ep_size: int | None = None):
-    import torch
-    dtype = dtype or (torch.bfloat16 if str(device).startswith("cuda")
-                      else torch.float32)
+    dtype = dtype or _dtype(device)
+    tp = dict(tp_rank=tp_rank, tp_size=tp_size, tp_group=tp_group)
+    if os.path.isfile(os.path.join(name, "config.json")):
+        return load_model(name, device=device, dtype=dtype, **tp)
+    if name.startswith("luzalorn") or name == "tiny-luzalorn":
+        from .luzalorn import LuzalornConfig, LuzalornModel
+        return LuzalornModel(LuzalornConfig.preset(name), device=device,
+                             dtype=dtype, seed=seed, **tp)
     if name.startswith("mixtral") or name == "tiny-moe":
         from .mixtral import MixtralConfig, MixtralModel
         return MixtralModel(MixtralConfig.preset(name), device=device,
-                            dtype=dtype, seed=seed, tp_rank=tp_rank,
-                            tp_size=tp_size, tp_group=tp_group,
-                            ep_size=ep_size)
+                            dtype=dtype, seed=seed, ep_size=ep_size, **tp)
     from .llama import LlamaConfig, LlamaModel
     return LlamaModel(LlamaConfig.preset(name), device=device, dtype=dtype,
-                      seed=seed, tp_rank=tp_rank, tp_size=tp_size,
-                      tp_group=tp_group)
+                      seed=seed, **tp)

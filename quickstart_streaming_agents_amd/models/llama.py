@@ -203,7 +203,9 @@ class LlamaModel:
                      self.tp_size)
         return {"wgu": wgu, "wdown": wdown}
 
-    def new_kv_cache(self, n_pages: int) -> PagedKVCache:
+    def new_kv_cache(self, n_pages: int,
+                     state_slots: int | None = None) -> PagedKVCache:
+        """state_slots: for decoders with recurrent layers; none here."""
         return PagedKVCache(self.cfg.n_layers, self.n_kv, self.cfg.d_head,
                             n_pages, self.device, self.dtype)
 
@@ -324,14 +326,17 @@ class LlamaModel:
 
     @torch.no_grad()
     def forward_prefill_batch(self, items: list[tuple[torch.Tensor, int, int]],
-                              kv: PagedKVCache) -> torch.Tensor:
+                              kv: PagedKVCache,
+                              want: list[list[int]] | None = None
+                              ) -> torch.Tensor:
         """Batched (and incremental) prefill.
 
         items: (new_tokens [t_i] i64, seq_id, start_pos).  start_pos > 0 means
         the sequence's first start_pos positions are already in the paged
         cache (prefix reuse across agent turns).  All per-token projections
         run as ONE fused GEMM over the concatenation; only attention loops
-        per sequence.  Returns last-position logits [n_items, vocab].
+        per sequence.  Returns the logits at the places `want` of every item
+        (default: its last position), in order.
         """
         c = self.cfg
         dev = self.device
@@ -472,8 +477,12 @@ class LlamaModel:
             h = D.rmsnorm_residual(o, res, L["mlp_norm"], c.norm_eps)
             mlp_out = self._ffn(L, h)
         final_h = D.rmsnorm_residual(mlp_out, res, self.final_norm, c.norm_eps)
-        last = torch.tensor([offs[i] + lens[i] - 1 for i in range(len(items))],
-                            dtype=torch.int64, device=dev)
+        if want is None:
+            want = [[n - 1] for n in lens]
+        last = torch.tensor([offs[i] + w for i, ws in enumerate(want)
+                             for w in ws], dtype=torch.int64, device=dev)
+        if not last.numel():
+            return final_h.new_empty(0, c.vocab_size)
         return self._linear(final_h.index_select(0, last), self.lm_head,
                             self.lm_head_f, self.lm_head_f8)
 

@@ -27,7 +27,7 @@ from dataclasses import dataclass, field
 
 import torch
 
-from .llama import LlamaModel
+from ..ops import dispatch as D
 
 
 @dataclass
@@ -46,6 +46,17 @@ class Sequence:
     decision_allowed: list[int] | None = None
     branches: dict[int, list[int]] | None = None
     script: list[int] | None = None
+
+
+@dataclass
+class StepEntry:
+    """What one live sequence contributes to a step: its next tokens, the
+    position of the first, and the places among them whose logits are asked
+    for."""
+    seq_id: int
+    tokens: list[int]
+    start: int
+    want: list[int]
 
 
 @dataclass
@@ -90,12 +101,14 @@ def _enable_tunableop() -> None:
 
 
 class Engine:
-    def __init__(self, model: LlamaModel, kv_pages: int | None = None,
+    def __init__(self, model, kv_pages: int | None = None,
                  max_batch: int = 256, max_seq_len: int = 4096,
                  eos_id: int | None = None, prefill_batch_tokens: int = 65536,
                  temperature: float = 0.0,
                  valid_vocab: tuple[int, int] | None = None,
-                 decision_temperature: float = 1.0):
+                 decision_temperature: float = 1.0,
+                 state_slots: int | None = None,
+                 chunk_tokens: int | None = None):
         if torch.cuda.is_available():
             _enable_tunableop()   # load the pre-tuned GEMM picks
         self.model = model
@@ -121,7 +134,17 @@ class Engine:
         self.prefill_batch_tokens = prefill_batch_tokens
         if kv_pages is None:
             kv_pages = max_batch * ((max_seq_len + 63) // 64) + 64
-        self.kv = model.new_kv_cache(kv_pages)
+        # state slots (recurrent layers): one per running sequence and one
+        # per conversation snapshot
+        self.kv = model.new_kv_cache(
+            kv_pages, state_slots=state_slots or 2 * max_batch)
+        if hasattr(model, "ensure_positions"):
+            model.ensure_positions(max_seq_len)
+        # chunked prefill: with chunk_tokens set, step() runs ONE mixed batch
+        # of every running sequence's next token and up to chunk_tokens
+        # prompt tokens, so a long prompt does not hold up decoding
+        self.chunk_tokens = chunk_tokens
+        self.reading: list[Sequence] = []    # prompts partly in the cache
         self._next_id = 0
         self.pending: list[Sequence] = []
         self.running: list[Sequence] = []
@@ -157,12 +180,11 @@ class Engine:
         if self._vocab_bias is not None:
             logits = logits.float() + self._vocab_bias
         if self.temperature <= 0.0:
-            return torch.argmax(logits, dim=-1)
+            return D.argmax_rows(logits)
         u = torch.rand(logits.shape, device=logits.device,
                        dtype=torch.float32).clamp_min_(1e-20)
         gumbel = -torch.log(-torch.log(u).clamp_min_(1e-20))
-        return torch.argmax(logits.float() + self.temperature * gumbel,
-                            dim=-1)
+        return D.argmax_rows(logits.float() + self.temperature * gumbel)
 
     def _sample_first(self, logits: torch.Tensor,
                       admitted: list["Sequence"]) -> list[int]:
@@ -231,6 +253,10 @@ class Engine:
             "script_mask": torch.zeros(B, self.MAX_RUN, dtype=torch.bool,
                                        device=dev),
         }
+        if self.kv.has_state:
+            # recurrent state slot of each row; -1: row not in use
+            gb["state_slots"] = torch.full((B,), -1, dtype=torch.int32,
+                                           device=dev)
 
         def body():
             # self-feeding decode step: advance seq_lens in-graph, append the
@@ -239,7 +265,8 @@ class Engine:
             positions = (gb["seq_lens"] - 1).clamp(min=0).int()
             logits = self.model.forward_decode(
                 gb["tokens"], self.kv, gb["block_table"], gb["seq_lens"],
-                positions)
+                positions, *([gb["state_slots"]] if self.kv.has_state
+                             else []))
             nxt = self._sample(logits)
             # grammar-forced tokens override the free sample in-graph
             j = gb["ctr"].clamp(max=self.MAX_RUN - 1)
@@ -282,9 +309,12 @@ class Engine:
         seq_ids = [s.seq_id for s in batch]
         bt = self.kv.block_table(seq_ids)
         sl = self.kv.seq_lens_tensor(seq_ids)
-        logits = self.model.forward_decode(tokens, self.kv, bt, sl,
-                                           positions)
-        nxt = self._sample(logits).tolist()
+        logits = self.model.forward_decode(
+            tokens, self.kv, bt, sl, positions,
+            *([self.kv.slots_tensor(seq_ids)] if self.kv.has_state else []))
+        self._push_decoded(batch, self._sample(logits).tolist())
+
+    def _push_decoded(self, batch: list[Sequence], nxt: list[int]) -> None:
         for s, tok in zip(batch, nxt):
             if s.script:
                 # grammar-forced continuation (script index: out_tokens[0]
@@ -331,6 +361,9 @@ class Engine:
         if n < self.max_batch:
             gb["seq_lens"][n:] = 0
             gb["active"][n:] = 0
+        if self.kv.has_state:
+            gb["state_slots"][:n] = self.kv.slots_tensor(seq_ids)
+            gb["state_slots"][n:] = -1
         # grammar scripts for this run window: run-step j emits
         # out_tokens[d + j] whose script index is d - 1 + j (out_tokens[0]
         # was the prefill-sampled decision token)
@@ -403,6 +436,7 @@ class Engine:
         if continue_from is not None:
             # at least one token must prefill (last-position logits)
             shared = min(len(continue_from.prompt), len(prompt) - 1)
+            shared = self.kv.reusable_prefix(continue_from.seq_id, shared)
             # shared prefix = the previous turn's prompt (its decode-token KV
             # is rolled back); bail to fresh prefill on any mismatch
             if prompt[:shared] != continue_from.prompt[:shared]:
@@ -413,6 +447,7 @@ class Engine:
                                decision_allowed=decision_allowed,
                                branches=branches)
                 self.kv.truncate(seq.seq_id, shared)
+                self.kv.claim(seq.seq_id)
                 self._next_id = max(self._next_id, seq.seq_id + 1)
                 self.pending.append(seq)
                 return seq
@@ -449,7 +484,7 @@ class Engine:
             have = len(self.kv._seq_pages.get(seq.seq_id, ())) \
                 if seq.cached_len else 0
             need = self.kv.pages_for(total) - have
-            if need > self.kv.free_pages:
+            if not self.kv.can_admit(seq.seq_id, need):
                 break
             delta = len(seq.prompt) - seq.cached_len
             if batch_items and new_tokens + delta > self.prefill_batch_tokens:
@@ -476,8 +511,17 @@ class Engine:
         if _TIMING:
             torch.cuda.synchronize()
             self.stats.prefill_s += time.perf_counter() - _t0
-        first = self._sample_first(logits, admitted)
         self.stats.prefill_batches += 1
+        self._start_decoding(admitted, logits)
+
+    def _start_decoding(self, admitted: list[Sequence],
+                        logits: torch.Tensor) -> None:
+        """Prompts fully read, one row of logits each: first token, grammar
+        branch, into the running batch."""
+        for seq in admitted:
+            if seq.keep_alive:
+                self.kv.snapshot(seq.seq_id)
+        first = self._sample_first(logits, admitted)
         for seq, tok in zip(admitted, first):
             seq.out_tokens.append(int(tok))
             if seq.branches is not None:
@@ -498,6 +542,103 @@ class Engine:
                         len(seq.script), room)
             self.running.append(seq)
             self._maybe_finish(seq)
+
+    # ---- one step over any mixture of portions and single tokens ---------
+    def step_entries(self, entries: list[StepEntry]) -> torch.Tensor:
+        """Run the entries as ONE batch; logits at the wanted places, in the
+        order of the entries.  A sequence is admitted with its first entry
+        (start 0) and goes on from wherever its cache and state are; its
+        pages grow as needed, kv.free() gives everything back.  Steps of
+        single tokens take the decode path."""
+        dev = self.model.device
+        for e in entries:
+            end = e.start + len(e.tokens)
+            if e.start == 0 and e.seq_id not in self.kv._seq_pages:
+                self.kv.allocate(e.seq_id, end)
+            else:
+                self.kv.extend(e.seq_id, max(end, self.kv.seq_len(e.seq_id)))
+        if all(len(e.tokens) == 1 for e in entries):
+            ids = [e.seq_id for e in entries]
+            pos = torch.tensor([e.start for e in entries], dtype=torch.int32,
+                               device=dev)
+            logits = self.model.forward_decode(
+                torch.tensor([e.tokens[0] for e in entries],
+                             dtype=torch.int64, device=dev),
+                self.kv, self.kv.block_table(ids), pos + 1, pos,
+                *([self.kv.slots_tensor(ids)] if self.kv.has_state else []))
+            rows = [i for i, e in enumerate(entries) for _ in e.want]
+            if rows == list(range(len(entries))):
+                return logits
+            return logits[torch.tensor(rows, dtype=torch.int64, device=dev)]
+        items = [(torch.tensor(e.tokens, dtype=torch.int64, device=dev),
+                  e.seq_id, e.start) for e in entries]
+        return self.model.forward_prefill_batch(
+            items, self.kv, want=[e.want for e in entries])
+
+    def _open_prompts(self) -> None:
+        """Move queued prompts into the set being read in portions."""
+        while self.pending and len(self.running) + len(self.reading) < \
+                self.max_batch:
+            seq = self.pending[0]
+            total = len(seq.prompt) + seq.max_new_tokens
+            have = len(self.kv._seq_pages.get(seq.seq_id, ())) \
+                if seq.cached_len else 0
+            if not self.kv.can_admit(seq.seq_id,
+                                     self.kv.pages_for(total) - have):
+                break
+            self.pending.pop(0)
+            if seq.cached_len:
+                self.kv.extend(seq.seq_id, len(seq.prompt))
+            else:
+                self.kv.allocate(seq.seq_id, len(seq.prompt))
+            self.stats.cached_prefix_tokens += seq.cached_len
+            self.stats.prefills += 1
+            self.reading.append(seq)
+
+    def _step_mixed(self) -> None:
+        """One batch: the next token of every running sequence and up to
+        chunk_tokens tokens of the prompts being read, oldest first."""
+        batch = [s for s in self.running if not s.done]
+        entries = [StepEntry(s.seq_id, [s.out_tokens[-1]],
+                             len(s.prompt) + len(s.out_tokens) - 1, [0])
+                   for s in batch]
+        budget, finished = self.chunk_tokens, []
+        for s in self.reading:
+            n = min(budget, len(s.prompt) - s.cached_len)
+            if n == 0:
+                break
+            budget -= n
+            last = s.cached_len + n == len(s.prompt)
+            entries.append(StepEntry(
+                s.seq_id, s.prompt[s.cached_len:s.cached_len + n],
+                s.cached_len, [n - 1] if last else []))
+            s.cached_len += n
+            self.stats.prefill_tokens += n
+            if last:
+                finished.append(s)
+        logits = self.step_entries(entries)
+        if batch:
+            self._push_decoded(batch, self._sample(logits[:len(batch)])
+                               .tolist())
+        self.stats.prefill_batches += 1
+        if finished:
+            self.reading = [s for s in self.reading if s not in finished]
+            self._start_decoding(finished, logits[len(batch):])
+
+    def _advance_mixed(self) -> bool:
+        """Chunked prefill: run a mixed step if any prompt is waiting or
+        being read; False when plain decoding is all that is left."""
+        if not self.chunk_tokens or not (self.pending or self.reading):
+            return False
+        self._open_prompts()
+        if not self.reading:
+            if not self.running:
+                raise MemoryError("decode stalled: pending prompts cannot be "
+                                  "admitted (KV pages exhausted?)")
+            return False
+        self._step_mixed()
+        self._retire()
+        return True
 
     def _maybe_finish(self, seq: Sequence) -> None:
         if len(seq.out_tokens) >= seq.max_new_tokens or (
@@ -529,13 +670,16 @@ class Engine:
         # NON-deterministically at bench scale — the prefill's H2D /
         # allocator traffic races the replaying graph's memory pool on
         # this stack — so admissions and decode run sequentially.
-        while self.pending:
+        for _ in range(max_run):
+            if not self._advance_mixed():
+                break
+        while self.pending and not self.chunk_tokens:
             before = len(self.pending)
             self._admit()
             if len(self.pending) == before:
                 break
         batch = [s for s in self.running if not s.done]
-        if batch:
+        if batch and not self.reading:
             run = min(min(s.max_new_tokens - len(s.out_tokens)
                           for s in batch), max_run, self.MAX_RUN)
             if run > 0:
@@ -544,14 +688,19 @@ class Engine:
                 else:
                     self._decode_run_eager(batch, run)
         self._retire()
-        if self.pending and not self.running and not batch:
+        if self.pending and not self.running and not batch \
+                and not self.reading:
             raise MemoryError("decode stalled: pending prompts cannot be "
                               "admitted (KV pages exhausted?)")
-        return len(self.running) + len(self.pending)
+        return len(self.running) + len(self.pending) + len(self.reading)
 
     def step(self) -> int:
-        """Admit + one decode step; returns remaining work count."""
-        self._admit()
+        """Admit + one decode step (or one mixed step under chunked
+        prefill); returns remaining work count."""
+        if self._advance_mixed():
+            return len(self.running) + len(self.pending) + len(self.reading)
+        if not self.chunk_tokens:
+            self._admit()
         batch = [s for s in self.running if not s.done]
         if not batch:
             self._retire()
@@ -571,11 +720,13 @@ class Engine:
         self.finished.clear()   # batch callers don't drain it
         t0 = time.perf_counter()
         if self.use_graph:
-            while self.pending or self.running:
+            while self.pending or self.running or self.reading:
+                if self._advance_mixed():
+                    continue
                 before = len(self.pending)
                 # drain the whole pending queue (possibly several prefill
                 # batches) before decoding: decode runs want the full batch
-                while self.pending:
+                while self.pending and not self.chunk_tokens:
                     n_before = len(self.pending)
                     self._admit()
                     if len(self.pending) == n_before:
@@ -595,10 +746,10 @@ class Engine:
                     self._decode_run_graph(batch, run)
                 self._retire()
         else:
-            while self.pending or self.running:
+            while self.pending or self.running or self.reading:
                 n_pending = len(self.pending)
                 remaining = self.step()
-                if remaining and not self.running and \
+                if remaining and not self.running and not self.reading and \
                         len(self.pending) == n_pending:
                     raise MemoryError(
                         "decode stalled: pending prompts cannot be "

@@ -102,3 +102,76 @@ def window_agg_ref(ts: torch.Tensor, key: torch.Tensor, value, t0: int,
         if value is not None:
             sums[key[i], w[i]] += float(value[i])
     return counts, sums
+
+
+# ---- mixer decoders --------------------------------------------------------
+
+def residual_norm_ref(res, y, table, ids, vec, w, b, eps, init, layer):
+    """In-place f32 residual update and its norm (dispatch.residual_norm)."""
+    if init:
+        res.zero_()
+    if y is not None:
+        res.add_(y.float())
+    if table is not None:
+        res.add_(table[ids].float())
+    if vec is not None:
+        res.add_(vec.float())
+    x = res
+    if layer:
+        x = x - x.mean(-1, keepdim=True)
+    x = x / torch.sqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+    if b is not None:
+        x = x + b.float()
+    return x.to(w.dtype)
+
+
+def latent_rows_ref(qa, cache, block_table, row_item, row_len, sink, window,
+                    scale):
+    R, H, KR = qa.shape[0], sink.numel(), cache.shape[2]
+    out = torch.zeros(R, H, KR)
+    flat = cache.reshape(-1, KR).float()
+    for r in range(R):
+        n = int(row_len[r])
+        if n <= 0:
+            continue
+        lo = max(0, n - window) if window > 0 else 0
+        pos = torch.arange(lo, n)
+        bt = block_table[int(row_item[r]) if row_item is not None else r]
+        c = flat[bt.long()[pos // 64] * 64 + pos % 64]
+        s = (qa[r].float().view(H, KR) @ c.T) * scale
+        p = torch.softmax(torch.cat([s, sink.float()[:, None]], 1), -1)
+        out[r] = p[:, :-1] @ c
+    return out.view(R, H * KR).to(qa.dtype)
+
+
+def retention_ref(x, cos_t, sin_t, decay, state, portions, out, rot, kscale,
+                  eps):
+    """portions: (slot, first row, first position, length); state and the
+    portions' rows of out are written."""
+    _, H, D, E = state.shape
+    half = rot // 2
+    for slot, r0, p0, n in portions:
+        rows = x[r0:r0 + n].float()
+        q = rows[:, :H * D].reshape(n, H, D).clone()
+        k = rows[:, H * D:2 * H * D].reshape(n, H, D).clone()
+        v = rows[:, 2 * H * D:2 * H * D + H * E].reshape(n, H, E)
+        g = rows[:, 2 * H * D + H * E:2 * H * D + 2 * H * E]
+        if half:
+            c = cos_t[p0:p0 + n, None, :]
+            s = sin_t[p0:p0 + n, None, :]
+            for t in (q, k):
+                a, b = t[..., :half].clone(), t[..., half:rot].clone()
+                t[..., :half] = a * c - b * s
+                t[..., half:rot] = b * c + a * s
+        k = k * kscale
+        S = state[slot]
+        if p0 == 0:
+            S.zero_()
+        o = torch.empty(n, H, E)
+        for t in range(n):
+            S.mul_(decay.view(H, 1, 1)).add_(k[t, :, :, None]
+                                             * v[t, :, None, :])
+            o[t] = torch.matmul(q[t, :, None, :], S).squeeze(1)
+        o = o / torch.sqrt(o.pow(2).mean(-1, keepdim=True) + eps)
+        out[r0:r0 + n] = (o.reshape(n, H * E)
+                          * torch.nn.functional.silu(g)).to(out.dtype)

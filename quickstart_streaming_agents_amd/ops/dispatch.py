@@ -1,7 +1,7 @@
 """Device dispatch for the op layer.
 
-Same call surface as the qsa_hip extension (ops/hip/ops.cpp). CUDA tensors
-go to the hand-written HIP/CDNA4 kernels — fail-loud if the extension is
+Same call surface as the native modules (ops/hip/ops.cpp: qsa_hip,
+ops/hip/lm_ops.cpp: qsa_lm_hip). CUDA tensors go to the hand-written HIP/CDNA4 kernels — fail-loud if the extension is
 missing (ops/__init__.py).  CPU tensors run reference implementations with
 IDENTICAL semantics (including in-place mutation contracts), which lets the
 engine / model / parallel layers run under multi-process gloo tests in
@@ -12,7 +12,7 @@ from __future__ import annotations
 
 import torch
 
-from . import ext
+from . import ext, lm_ext
 
 
 def _cuda(t: torch.Tensor) -> bool:
@@ -167,8 +167,6 @@ def can_pack_weight(n: int, k: int) -> bool:
 
 def pack_weight_frag(w: torch.Tensor) -> torch.Tensor:
     """[N,K] bf16 -> fragment-major stream layout for skinny_linear (GPU)."""
-    if w.is_cuda:
-        return ext().pack_weight_frag(w)
     n, k = w.shape
     return w.reshape(n // 16, 16, k // 32, 32).permute(0, 2, 1, 3).contiguous()
 
@@ -177,7 +175,7 @@ def skinny_linear(x: torch.Tensor, wf: torch.Tensor, n: int,
                   k: int) -> torch.Tensor:
     """x[M,K] @ W^T via the weight-streaming decode kernel (M <= 32)."""
     if x.is_cuda:
-        return ext().skinny_gemm(x, wf, n, k)
+        return lm_ext().skinny_gemm(x, wf, n, k)
     w = wf.reshape(n // 16, k // 32, 16, 32).permute(0, 2, 1, 3) \
         .reshape(n, k)
     return (x.float() @ w.float().T).to(x.dtype)
@@ -224,6 +222,153 @@ def skinny_linear_fp8(x: torch.Tensor, qf: torch.Tensor,
         return ext().skinny_gemm_fp8(x, qf, scale, n, k)
     w = unpack_weight_fp8(qf, scale, n, k)
     return (x.float() @ w.T).to(x.dtype)
+
+
+# ---- mixer decoders (qsa_lm_hip) ------------------------------------------
+# bf16 or f32 storage, f32 arithmetic, any sizes; the CPU semantics are in
+# ops/cpu_ref.py.
+
+def residual_norm(res: torch.Tensor, y: torch.Tensor | None,
+                  w: torch.Tensor, b: torch.Tensor | None, eps: float, *,
+                  table: torch.Tensor | None = None,
+                  ids: torch.Tensor | None = None,
+                  vec: torch.Tensor | None = None, init: bool = False,
+                  layer: bool = True) -> torch.Tensor:
+    """res (f32) <- (0 if init else res) + y + table[ids] + vec, in place;
+    returns the layer norm (layer=True) or rms norm of it, times w, plus b."""
+    if _cuda(res):
+        return lm_ext().residual_norm(res, y, table, ids, vec, w, b, eps,
+                                      init, layer)
+    from .cpu_ref import residual_norm_ref
+    return residual_norm_ref(res, y, table, ids, vec, w, b, eps, init, layer)
+
+
+def glu(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
+    """silu(gate) * up for any width and storage type."""
+    if _cuda(gate):
+        return lm_ext().glu(gate, up)
+    return (torch.nn.functional.silu(gate.float()) * up.float()).to(gate.dtype)
+
+
+def argmax_rows(x: torch.Tensor) -> torch.Tensor:
+    """Greedy pick per row (lowest index on ties), safe inside graphs."""
+    if _cuda(x):
+        return lm_ext().argmax_rows(x.contiguous())
+    return torch.argmax(x, dim=-1)
+
+
+def decode_slots(block_table: torch.Tensor,
+                 seq_lens: torch.Tensor) -> torch.Tensor:
+    """Cache slot (page*64 + offset) of each row's newest position, or -1."""
+    if _cuda(block_table):
+        return lm_ext().decode_slots(block_table, seq_lens)
+    p = seq_lens.long() - 1
+    pc = p.clamp(min=0)
+    page = block_table.long().gather(1, (pc // 64)[:, None]).squeeze(1)
+    return torch.where(p < 0, torch.full_like(p, -1),
+                       page * 64 + pc % 64).int()
+
+
+def latent_norm_store(x: torch.Tensor, wq: torch.Tensor, wk: torch.Tensor,
+                      cache: torch.Tensor, slots: torch.Tensor,
+                      eps: float) -> torch.Tensor:
+    """x rows [q latent | kv latent | ...]: returns rms(q latent) * wq and
+    writes rms(kv latent) * wk to cache [pages, 64, rank] at `slots`."""
+    if _cuda(x):
+        return lm_ext().latent_norm_store(x, wq, wk, cache, slots, eps)
+    from .cpu_ref import rmsnorm_ref
+    qr, kr = wq.numel(), wk.numel()
+    c = rmsnorm_ref(x[:, qr:qr + kr], wk, eps).to(cache.dtype)
+    keep = slots >= 0
+    cache.view(-1, kr)[slots[keep].long()] = c[keep]
+    return rmsnorm_ref(x[:, :qr], wq, eps).to(x.dtype)
+
+
+def head_matmul(x: torch.Tensor, w: torch.Tensor,
+                gate: torch.Tensor | None = None) -> torch.Tensor:
+    """x [M, H*K], w [H, N, K] -> [M, H*N], one product per head; with
+    `gate` [M, H*N] the result is multiplied by sigmoid(gate)."""
+    if _cuda(x):
+        return lm_ext().head_matmul(x, w, gate)
+    H, N, K = w.shape
+    y = torch.bmm(x.float().reshape(-1, H, K).transpose(0, 1).contiguous(),
+                  w.float().transpose(1, 2).contiguous())
+    y = y.transpose(0, 1).reshape(-1, H * N)
+    if gate is not None:
+        y = y * torch.sigmoid(gate.float())
+    return y.to(x.dtype)
+
+
+def latent_rows(qa: torch.Tensor, cache: torch.Tensor,
+                block_table: torch.Tensor, row_item: torch.Tensor | None,
+                row_len: torch.Tensor, sink: torch.Tensor, window: int,
+                scale: float) -> torch.Tensor:
+    """Absorbed latent attention: row r of qa [R, H*rank] at position
+    row_len[r]-1 reads the latents of sequence row_item[r] (its own index
+    without it) inside the window (0: all); softmax with sink."""
+    if _cuda(qa):
+        return lm_ext().latent_rows(qa, cache, block_table, row_item,
+                                    row_len, sink, window, scale)
+    from .cpu_ref import latent_rows_ref
+    return latent_rows_ref(qa, cache, block_table, row_item, row_len, sink,
+                           window, scale)
+
+
+def window_attn_ok(h: int, d: int, e: int) -> bool:
+    return lm_ext().window_attn_ok(h, d, e)
+
+
+def window_attn_prefill(q, kv, gate, sink, qb_item, qb_t0, off, start, len_,
+                        ctx_off, ctx_pos, out, d: int, e: int, window: int,
+                        scale: float) -> None:
+    """Windowed flash attention of prompt portions over expanded keys and
+    values, sink and sigmoid gate included (GPU, bf16)."""
+    lm_ext().window_attn_prefill(q, kv, gate, sink, qb_item, qb_t0, off,
+                                 start, len_, ctx_off, ctx_pos, out, d, e,
+                                 window, scale)
+
+
+def retention_decode(x, cos_t, sin_t, decay, state, slots, seq_lens,
+                     rot: int, kscale: float, eps: float) -> torch.Tensor:
+    """One token per row; x rows [q | k | v | gate], state [slots, H, D, E]
+    f32 updated in place.  Rows with seq_len 0 or slot -1 are not in use."""
+    if _cuda(x):
+        return lm_ext().retention_decode(x, cos_t, sin_t, decay, state,
+                                         slots, seq_lens, rot, kscale, eps)
+    from .cpu_ref import retention_ref
+    B, (_, H, D, E) = x.shape[0], state.shape
+    out = torch.zeros(B, H * E, dtype=x.dtype)
+    live = [b for b in range(B) if int(seq_lens[b]) > 0 and int(slots[b]) >= 0]
+    retention_ref(x, cos_t, sin_t, decay, state,
+                  [(int(slots[b]), b, int(seq_lens[b]) - 1, 1) for b in live],
+                  out, rot, kscale, eps)
+    return out
+
+
+def retention_seq(x, cos_t, sin_t, decay, state, slots, off, start, len_,
+                  out, rot: int, kscale: float, eps: float) -> None:
+    """Portions of several tokens, token by token (any size and type)."""
+    if _cuda(x):
+        lm_ext().retention_seq(x, cos_t, sin_t, decay, state, slots, off,
+                               start, len_, out, rot, kscale, eps)
+        return
+    from .cpu_ref import retention_ref
+    retention_ref(x, cos_t, sin_t, decay, state,
+                  list(zip(slots.tolist(), off.tolist(), start.tolist(),
+                           len_.tolist())), out, rot, kscale, eps)
+
+
+def retention_chunked_ok(h: int, d: int, e: int) -> bool:
+    return lm_ext().retention_chunked_ok(h, d, e)
+
+
+def retention_chunked(x, cos_t, sin_t, log2_decay, state, slots, off, start,
+                      len_, positions, chunk0, chunk_item, chunk_t0, out,
+                      rot: int, kscale: float, eps: float) -> None:
+    """Portions in chunks of 64 tokens on the matrix cores (GPU, bf16)."""
+    lm_ext().retention_chunked(x, cos_t, sin_t, log2_decay, state, slots,
+                               off, start, len_, positions, chunk0,
+                               chunk_item, chunk_t0, out, rot, kscale, eps)
 
 
 # ---- retrieval / streaming ------------------------------------------------

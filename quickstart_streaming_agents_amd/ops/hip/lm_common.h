@@ -1,0 +1,107 @@
+// Shared device helpers of the decoder-mixer kernels (qsa_lm_hip).
+//
+// Every scalar kernel is a template over the storage type T: bf16 (held as
+// unsigned short) or float.  All arithmetic is f32; T is only how operands
+// and results are stored.
+#pragma once
+
+#include "common.h"
+
+typedef unsigned short bf16_t;
+
+using bf16x8_v = __attribute__((ext_vector_type(8))) short;
+using bf16x4_v = __attribute__((ext_vector_type(4))) short;
+using f32x4_v = __attribute__((ext_vector_type(4))) float;
+
+template <typename T> __device__ __forceinline__ float ldf(const T* p);
+template <> __device__ __forceinline__ float ldf<bf16_t>(const bf16_t* p) {
+  return bf16_to_f32(*p);
+}
+template <> __device__ __forceinline__ float ldf<float>(const float* p) {
+  return *p;
+}
+template <typename T> __device__ __forceinline__ void stf(T* p, float v);
+template <> __device__ __forceinline__ void stf<bf16_t>(bf16_t* p, float v) {
+  *p = f32_to_bf16(v);
+}
+template <> __device__ __forceinline__ void stf<float>(float* p, float v) {
+  *p = v;
+}
+
+// VEC consecutive elements <-> f32 registers (pointer aligned to the group)
+template <typename T, int VEC>
+__device__ __forceinline__ void ldv(const T* p, float* v) {
+  if constexpr (VEC == 1) {
+    v[0] = ldf<T>(p);
+  } else if constexpr (sizeof(T) == 4) {
+#pragma unroll
+    for (int i = 0; i < VEC; i += 4) {
+      const float4 f = *reinterpret_cast<const float4*>(p + i);
+      v[i] = f.x; v[i + 1] = f.y; v[i + 2] = f.z; v[i + 3] = f.w;
+    }
+  } else {
+#pragma unroll
+    for (int i = 0; i < VEC; i += 4) {
+      const uint2 u = *reinterpret_cast<const uint2*>(p + i);
+      const float2 a = bf16x2_to_f32x2(u.x), b = bf16x2_to_f32x2(u.y);
+      v[i] = a.x; v[i + 1] = a.y; v[i + 2] = b.x; v[i + 3] = b.y;
+    }
+  }
+}
+template <typename T, int VEC>
+__device__ __forceinline__ void stv(T* p, const float* v) {
+  if constexpr (VEC == 1) {
+    stf<T>(p, v[0]);
+  } else if constexpr (sizeof(T) == 4) {
+#pragma unroll
+    for (int i = 0; i < VEC; i += 4)
+      *reinterpret_cast<float4*>(p + i) =
+          make_float4(v[i], v[i + 1], v[i + 2], v[i + 3]);
+  } else {
+#pragma unroll
+    for (int i = 0; i < VEC; i += 4)
+      *reinterpret_cast<uint2*>(p + i) = make_uint2(
+          f32x2_to_bf16x2(v[i], v[i + 1]), f32x2_to_bf16x2(v[i + 2], v[i + 3]));
+  }
+}
+
+__device__ __forceinline__ float silu_f(float z) { return z / (1.f + expf(-z)); }
+__device__ __forceinline__ float sigmoid_f(float z) {
+  return 1.f / (1.f + expf(-z));
+}
+
+// x = hi + lo with both parts bf16: 16 mantissa bits survive, so a product
+// of two such pairs on the bf16 matrix cores (hi*hi + hi*lo + lo*hi) stays
+// at f32-like accuracy.
+__device__ __forceinline__ void split_bf16(float x, bf16_t& hi, bf16_t& lo) {
+  hi = f32_to_bf16(x);
+  lo = f32_to_bf16(x - bf16_to_f32(hi));
+}
+
+// Transposing LDS read: within 16 lanes, lane i supplies the address of 4
+// consecutive elements of row i/4, columns (i%4)*4.. of a 4 x 16 block and
+// receives column i, i.e. 4 consecutive rows of one column.
+__device__ __forceinline__ bf16x4_v lds_read_tr(const bf16_t* p) {
+  typedef __attribute__((address_space(3))) bf16x4_v* lds_ptr;
+  return __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_ptr)p);
+}
+
+// Two transposed 4-row groups of column `col_tile*16 + lane%16` as one
+// 8-element MFMA operand: rows row0 + hi*4 .. +3 and row1 + hi*4 .. +3
+// (hi = lane / 16).
+__device__ __forceinline__ bf16x8_v lds_frag_tr(const bf16_t* tile, int pitch,
+                                                int row0, int row1, int col0,
+                                                int lane) {
+  const int r = (lane >> 4) * 4 + ((lane & 15) >> 2);
+  const int c = col0 + (lane & 3) * 4;
+  const bf16x4_v a = lds_read_tr(tile + (row0 + r) * pitch + c);
+  const bf16x4_v b = lds_read_tr(tile + (row1 + r) * pitch + c);
+  return __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7);
+}
+
+__device__ __forceinline__ f32x4_v mfma_bf16(bf16x8_v a, bf16x8_v b,
+                                             f32x4_v c) {
+  typedef __attribute__((ext_vector_type(8))) __bf16 raw;
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+      __builtin_bit_cast(raw, a), __builtin_bit_cast(raw, b), c, 0, 0, 0);
+}
