@@ -53,6 +53,12 @@ def parse_args():
     p.add_argument("--decode-chunk", type=int, default=8,
                    help="decode steps per engine slice in the continuous "
                         "scheduler")
+    p.add_argument("--workload", default="lab1",
+                   choices=("lab1", "luzalorn", "luzalorn-kernels",
+                            "luzalorn-models"),
+                   help="lab1: the headline benchmark (default); luzalorn: "
+                        "prefill/decode throughput and kernel rooflines of "
+                        "that design beside the Llama decoder")
     p.add_argument("--stub-llm", action="store_true",
                    help="CPU contract check: stub LLM instead of the GPU engine")
     return p.parse_args()
@@ -60,6 +66,10 @@ def parse_args():
 
 def main():
     args = parse_args()
+    if args.workload != "lab1":
+        from quickstart_streaming_agents_amd.models import bench as models_bench
+        models_bench.main(args.workload.partition("-")[2] or "all")
+        return
     import torch
 
     world = int(os.environ.get("WORLD_SIZE", "1"))

@@ -5,6 +5,8 @@ surface (pyproject.toml:90-165) on the local MI355X engine.
     python -m quickstart_streaming_agents_amd run     --lab 1 [--device cuda]
     python -m quickstart_streaming_agents_amd datagen --lab 3
     python -m quickstart_streaming_agents_amd validate
+    python -m quickstart_streaming_agents_amd generate --model DIR --tokens 1,2
+    python -m quickstart_streaming_agents_amd replay --model DIR --out OUT ...
     python -m quickstart_streaming_agents_amd destroy --dir out
 """
 
@@ -232,6 +234,41 @@ def cmd_serve(args) -> int:
                       (["--model", args.model] if args.model else []))
 
 
+def cmd_generate(args) -> int:
+    """Continue prompts with a model: a preset name (random weights) or a
+    folder with config.json and model.safetensors."""
+    from .models import build_model
+    from .models.serve import Engine
+    from .models.tokenizer import default_tokenizer
+    model = build_model(args.model, device=args.device)
+    tok = None
+    if args.tokens:
+        prompts = [[int(t) for t in p.split(",")] for p in args.tokens]
+    elif args.prompt:
+        tok = default_tokenizer(model.cfg.vocab_size)
+        prompts = [tok.encode(p) for p in args.prompt]
+    else:
+        print("generate: give --prompt or --tokens", file=sys.stderr)
+        return 2
+    longest = max(len(p) for p in prompts) + args.max_new
+    engine = Engine(model, max_batch=len(prompts), max_seq_len=longest,
+                    temperature=args.temperature,
+                    chunk_tokens=args.chunk_tokens)
+    for p, out in zip(prompts, engine.generate_batch(
+            prompts, [args.max_new] * len(prompts))):
+        print(json.dumps({"prompt_tokens": len(p), "tokens": out,
+                          **({"text": tok.decode(out)} if tok else {})}))
+    return 0
+
+
+def cmd_replay(args) -> int:
+    from .models.replay import main as replay_main
+    return replay_main(["--model", args.model, "--dtype", args.dtype,
+                        "--out", args.out,
+                        "--max-tokens", str(args.max_tokens)] +
+                       (["--device", args.device] if args.device else []))
+
+
 def cmd_tests(args) -> int:
     import os
     import subprocess
@@ -322,6 +359,30 @@ def main(argv=None) -> int:
     s.add_argument("--device", default="cpu")
     s.add_argument("--model", default=None)
     s.set_defaults(fn=cmd_serve)
+
+    n = sub.add_parser("generate", help="continue prompts with a model "
+                       "(preset name or checkpoint folder)")
+    n.add_argument("--model", required=True)
+    n.add_argument("--prompt", action="append", help="text (repeatable)")
+    n.add_argument("--tokens", action="append",
+                   help="comma-separated token ids (repeatable)")
+    n.add_argument("--max-new", type=int, default=32)
+    n.add_argument("--temperature", type=float, default=0.0)
+    n.add_argument("--chunk-tokens", type=int, default=None,
+                   help="read prompts in portions of at most this many "
+                        "tokens a step, beside running decodes")
+    n.add_argument("--device", default="cuda:0")
+    n.set_defaults(fn=cmd_generate)
+
+    y = sub.add_parser("replay", help="feed a token trace (JSON lines on "
+                       "stdin) through a model and write logits")
+    y.add_argument("--model", required=True)
+    y.add_argument("--dtype", choices=("bfloat16", "float32"),
+                   default="bfloat16")
+    y.add_argument("--out", required=True)
+    y.add_argument("--max-tokens", type=int, required=True)
+    y.add_argument("--device", default=None)
+    y.set_defaults(fn=cmd_replay)
 
     t = sub.add_parser("tests", help="run the test suite "
                        "(scripts/run_tests.py parity)")

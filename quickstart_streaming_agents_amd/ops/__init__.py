@@ -37,7 +37,7 @@ def lm_ext():
     if _lm_ext is None:
         raise RuntimeError(
             "qsa_lm_hip extension not built. Run "
-            "`PYTORCH_ROCM_ARCH=gfx950 python setup.py build_ext --inplace` "
+            "`python setup.py build_ext --inplace` "
             f"(import error: {_lm_import_error})")
     return _lm_ext
 
@@ -51,6 +51,6 @@ def ext():
     if _ext is None:
         raise RuntimeError(
             "qsa_hip extension not built. Run "
-            "`PYTORCH_ROCM_ARCH=gfx950 python setup.py build_ext --inplace` "
+            "`python setup.py build_ext --inplace` "
             f"(import error: {_import_error})")
     return _ext

@@ -327,7 +327,7 @@ qsa_latent_rows_mfma(const bf16_t* __restrict__ qa,
         p[r] = s4[r] > NEG_BIG ? exp2f(s4[r] - mn) : 0.f;
       l = l * alpha + (p[0] + p[1]) + (p[2] + p[3]);
       ps[wave][lane] =
-          make_uint2(f32x2_to_bf16x2(p[0], p[1]), f32x2_to_bf16x2(p[2], p[3]));
+          make_uint2(cvt_bf16x2(p[0], p[1]), cvt_bf16x2(p[2], p[3]));
 #pragma unroll
       for (int t = 0; t < DTW; ++t) acc[t] *= alpha;
       __syncthreads();
@@ -561,7 +561,7 @@ qsa_window_attn_prefill(const bf16_t* __restrict__ q, long long qstride,
       for (int r = 0; r < 4; ++r) {
         const float p = s4[pt][r] > NEG_BIG ? exp2f(s4[pt][r] - mn) : 0.f;
         psum += p;
-        pf[pt >> 1][(pt & 1) * 4 + r] = (short)f32_to_bf16(p);
+        pf[pt >> 1][(pt & 1) * 4 + r] = (short)cvt_bf16(p);
       }
     l = l * alpha + psum;
 #pragma unroll
@@ -570,7 +570,6 @@ qsa_window_attn_prefill(const bf16_t* __restrict__ q, long long qstride,
     for (int s = 0; s < 2; ++s)
 #pragma unroll
       for (int t = 0; t < ET; ++t) {
-        if (t * 16 >= E) break;                     // uniform
         const bf16x8_v a =
             lds_frag_tr(vt, VP, s * 32, s * 32 + 16, t * 16, lane);
         acc[t] = mfma_bf16(a, pf[s], acc[t]);

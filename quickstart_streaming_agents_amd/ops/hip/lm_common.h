@@ -11,7 +11,19 @@ typedef unsigned short bf16_t;
 
 using bf16x8_v = __attribute__((ext_vector_type(8))) short;
 using bf16x4_v = __attribute__((ext_vector_type(4))) short;
+using u32x4_v = __attribute__((ext_vector_type(4))) unsigned int;
 using f32x4_v = __attribute__((ext_vector_type(4))) float;
+
+// round-to-nearest-even with the hardware's packed conversion
+__device__ __forceinline__ unsigned int cvt_bf16x2(float a, float b) {
+  typedef __attribute__((ext_vector_type(2))) float f2;
+  typedef __attribute__((ext_vector_type(2))) __bf16 b2;
+  return __builtin_bit_cast(unsigned int,
+                            __builtin_convertvector((f2){a, b}, b2));
+}
+__device__ __forceinline__ bf16_t cvt_bf16(float a) {
+  return __builtin_bit_cast(bf16_t, (__bf16)a);
+}
 
 template <typename T> __device__ __forceinline__ float ldf(const T* p);
 template <> __device__ __forceinline__ float ldf<bf16_t>(const bf16_t* p) {
@@ -22,7 +34,7 @@ template <> __device__ __forceinline__ float ldf<float>(const float* p) {
 }
 template <typename T> __device__ __forceinline__ void stf(T* p, float v);
 template <> __device__ __forceinline__ void stf<bf16_t>(bf16_t* p, float v) {
-  *p = f32_to_bf16(v);
+  *p = cvt_bf16(v);
 }
 template <> __device__ __forceinline__ void stf<float>(float* p, float v) {
   *p = v;
@@ -61,7 +73,7 @@ __device__ __forceinline__ void stv(T* p, const float* v) {
 #pragma unroll
     for (int i = 0; i < VEC; i += 4)
       *reinterpret_cast<uint2*>(p + i) = make_uint2(
-          f32x2_to_bf16x2(v[i], v[i + 1]), f32x2_to_bf16x2(v[i + 2], v[i + 3]));
+          cvt_bf16x2(v[i], v[i + 1]), cvt_bf16x2(v[i + 2], v[i + 3]));
   }
 }
 
@@ -74,8 +86,17 @@ __device__ __forceinline__ float sigmoid_f(float z) {
 // of two such pairs on the bf16 matrix cores (hi*hi + hi*lo + lo*hi) stays
 // at f32-like accuracy.
 __device__ __forceinline__ void split_bf16(float x, bf16_t& hi, bf16_t& lo) {
-  hi = f32_to_bf16(x);
-  lo = f32_to_bf16(x - bf16_to_f32(hi));
+  hi = cvt_bf16(x);
+  lo = cvt_bf16(x - bf16_to_f32(hi));
+}
+
+// four values -> their packed hi and lo parts
+__device__ __forceinline__ void split4_bf16(float a, float b, float c, float d,
+                                            uint2& hi, uint2& lo) {
+  hi = make_uint2(cvt_bf16x2(a, b), cvt_bf16x2(c, d));
+  const float2 h0 = bf16x2_to_f32x2(hi.x), h1 = bf16x2_to_f32x2(hi.y);
+  lo = make_uint2(cvt_bf16x2(a - h0.x, b - h0.y),
+                  cvt_bf16x2(c - h1.x, d - h1.y));
 }
 
 // Transposing LDS read: within 16 lanes, lane i supplies the address of 4

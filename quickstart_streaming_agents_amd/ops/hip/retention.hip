@@ -269,23 +269,21 @@ qsa_retention_rotate(const bf16_t* __restrict__ x, long long xstride,
     const float* sn = sin_t + (long long)p * (rot >> 1);
     const bf16_t* q = x + row * xstride + (long long)h * D;
     const bf16_t* k = q + (long long)H * D;
-    bf16_t qh[4], ql[4], kh[4], kl[4];
+    float qv[4], kv[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int d = d0 + j;
-      const float qv = d < D ? rot_elem<bf16_t>(q, d, rot, cs, sn) : 0.f;
-      const float kv =
-          d < D ? rot_elem<bf16_t>(k, d, rot, cs, sn) * kscale : 0.f;
-      split_bf16(qv, qh[j], ql[j]);
-      split_bf16(kv, kh[j], kl[j]);
+      qv[j] = d < D ? rot_elem<bf16_t>(q, d, rot, cs, sn) : 0.f;
+      kv[j] = d < D ? rot_elem<bf16_t>(k, d, rot, cs, sn) * kscale : 0.f;
     }
-    const long long o = rh * DP + d0;
-    auto put = [&](long long base, const bf16_t* v) {
-      *reinterpret_cast<uint2*>(planes + base + o) =
-          make_uint2((unsigned)v[0] | ((unsigned)v[1] << 16),
-                     (unsigned)v[2] | ((unsigned)v[3] << 16));
-    };
-    put(0, qh); put(plane, ql); put(2 * plane, kh); put(3 * plane, kl);
+    uint2 a, b;
+    bf16_t* o = planes + rh * DP + d0;
+    split4_bf16(qv[0], qv[1], qv[2], qv[3], a, b);
+    *reinterpret_cast<uint2*>(o) = a;
+    *reinterpret_cast<uint2*>(o + plane) = b;
+    split4_bf16(kv[0], kv[1], kv[2], kv[3], a, b);
+    *reinterpret_cast<uint2*>(o + 2 * plane) = a;
+    *reinterpret_cast<uint2*>(o + 3 * plane) = b;
   }
 }
 
@@ -347,66 +345,58 @@ qsa_retention_state(const bf16_t* __restrict__ x, long long xstride,
       acc[t][r] = (p0 > 0 && d < D && e < E) ? S[(long long)d * E + e] : 0.f;
     }
 
-  uint4 kreg[2][KLD], vreg[2];
-  auto fetch = [&](int t0) {
-#pragma unroll
-    for (int p = 0; p < 2; ++p)
-#pragma unroll
-      for (int u = 0; u < KLD; ++u) {
-        const int g = tid + u * 256;
-        const int row = g / (DP / 8), c = (g % (DP / 8)) * 8;
-        const int tr = min(t0 + row, n - 1);
-        kreg[p][u] = *reinterpret_cast<const uint4*>(
-            kpl + p * plane + ((long long)(r0 + tr) * H + h) * DP + c);
-      }
-#pragma unroll
-    for (int u = 0; u < 2; ++u) {
-      const int g = tid + u * 256;
-      const int row = g >> 3, c = v0 + (g & 7) * 8;
-      const int tr = min(t0 + row, n - 1);
-      const int cc = min(c, E - 8);            // E % 8 == 0
-      vreg[u] = *reinterpret_cast<const uint4*>(
-          x + (long long)(r0 + tr) * xstride + voff + (long long)h * E + cc);
-    }
-  };
-  fetch(0);
+  u32x4_v kh[KLD], kl[KLD], vreg[2];
+#define QSA_FETCH(t0_)                                                        \
+  {                                                                           \
+    _Pragma("unroll") for (int u = 0; u < KLD; ++u) {                         \
+      const int g = tid + u * 256;                                            \
+      const int tr = min((t0_) + g / (DP / 8), n - 1);                        \
+      const bf16_t* src = kpl + ((long long)(r0 + tr) * H + h) * DP +         \
+                          (g % (DP / 8)) * 8;                                 \
+      kh[u] = *reinterpret_cast<const u32x4_v*>(src);                           \
+      kl[u] = *reinterpret_cast<const u32x4_v*>(src + plane);                   \
+    }                                                                         \
+    _Pragma("unroll") for (int u = 0; u < 2; ++u) {                           \
+      const int g = tid + u * 256;                                            \
+      const int tr = min((t0_) + (g >> 3), n - 1);                            \
+      const int cc = min(v0 + (g & 7) * 8, E - 8); /* E % 8 == 0 */           \
+      vreg[u] = *reinterpret_cast<const u32x4_v*>(                              \
+          x + (long long)(r0 + tr) * xstride + voff + (long long)h * E + cc); \
+    }                                                                         \
+  }
+  QSA_FETCH(0)
   const int nc = (n + RC - 1) / RC;
   for (int c = 0; c < nc; ++c) {
     const int t0 = c * RC;
     const int m = min(RC, n - t0);
     __syncthreads();                 // previous chunk's LDS readers are done
 #pragma unroll
-    for (int p = 0; p < 2; ++p)
-#pragma unroll
-      for (int u = 0; u < KLD; ++u) {
-        const int g = tid + u * 256;
-        const int row = g / (DP / 8), cc = (g % (DP / 8)) * 8;
-        *reinterpret_cast<uint4*>(&kt[p][row * KP + cc]) = kreg[p][u];
-      }
+    for (int u = 0; u < KLD; ++u) {
+      const int g = tid + u * 256;
+      const int o = g / (DP / 8) * KP + (g % (DP / 8)) * 8;
+      *reinterpret_cast<u32x4_v*>(&kt[0][o]) = kh[u];
+      *reinterpret_cast<u32x4_v*>(&kt[1][o]) = kl[u];
+    }
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
       const int g = tid + u * 256;
       const int row = g >> 3, cc = (g & 7) * 8;
       const bool ok = row < m && v0 + cc < E;
-      const float f = ok ? exp2f((float)(m - 1 - row) * l2d) : 0.f;
-      const unsigned pk[4] = {vreg[u].x, vreg[u].y, vreg[u].z, vreg[u].w};
-      unsigned oh[4], ol[4];
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const float2 v = bf16x2_to_f32x2(pk[j]);
-        bf16_t h0, l0, h1, l1;
-        split_bf16(ok ? v.x * f : 0.f, h0, l0);
-        split_bf16(ok ? v.y * f : 0.f, h1, l1);
-        oh[j] = (unsigned)h0 | ((unsigned)h1 << 16);
-        ol[j] = (unsigned)l0 | ((unsigned)l1 << 16);
-      }
+      const float f = exp2f((float)(m - 1 - row) * l2d);
+      const u32x4_v pk = ok ? vreg[u] : (u32x4_v){0, 0, 0, 0};
+      const float fo = ok ? f : 0.f;
+      const float2 v01 = bf16x2_to_f32x2(pk.x), v23 = bf16x2_to_f32x2(pk.y);
+      const float2 v45 = bf16x2_to_f32x2(pk.z), v67 = bf16x2_to_f32x2(pk.w);
+      uint2 h0, l0, h1, l1;
+      split4_bf16(v01.x * fo, v01.y * fo, v23.x * fo, v23.y * fo, h0, l0);
+      split4_bf16(v45.x * fo, v45.y * fo, v67.x * fo, v67.y * fo, h1, l1);
       *reinterpret_cast<uint4*>(&vt[0][row * VP + cc]) =
-          make_uint4(oh[0], oh[1], oh[2], oh[3]);
+          make_uint4(h0.x, h0.y, h1.x, h1.y);
       *reinterpret_cast<uint4*>(&vt[1][row * VP + cc]) =
-          make_uint4(ol[0], ol[1], ol[2], ol[3]);
+          make_uint4(l0.x, l0.y, l1.x, l1.y);
     }
     __syncthreads();
-    if (c + 1 < nc) fetch(t0 + RC);
+    if (c + 1 < nc) QSA_FETCH(t0 + RC)
 
     // state before this chunk (nothing precedes the first token)
     if ((c > 0 || p0 > 0) && e < EP) {
@@ -415,16 +405,11 @@ qsa_retention_state(const bf16_t* __restrict__ x, long long xstride,
       bf16_t* pl = ph + n_chunks * H * EP * DP;
 #pragma unroll
       for (int t = 0; t < 2 * KS; ++t) {
-        bf16_t a[4], b[4];
-#pragma unroll
-        for (int r = 0; r < 4; ++r) split_bf16(acc[t][r], a[r], b[r]);
+        uint2 a, b;
+        split4_bf16(acc[t][0], acc[t][1], acc[t][2], acc[t][3], a, b);
         const int d = t * 16 + hi * 4;
-        *reinterpret_cast<uint2*>(ph + d) =
-            make_uint2((unsigned)a[0] | ((unsigned)a[1] << 16),
-                       (unsigned)a[2] | ((unsigned)a[3] << 16));
-        *reinterpret_cast<uint2*>(pl + d) =
-            make_uint2((unsigned)b[0] | ((unsigned)b[1] << 16),
-                       (unsigned)b[2] | ((unsigned)b[3] << 16));
+        *reinterpret_cast<uint2*>(ph + d) = a;
+        *reinterpret_cast<uint2*>(pl + d) = b;
       }
     }
     const float dn = exp2f((float)m * l2d);
@@ -456,6 +441,8 @@ qsa_retention_state(const bf16_t* __restrict__ x, long long xstride,
       if (d < D && e < E) S[(long long)d * E + e] = acc[t][r];
     }
 }
+
+#undef QSA_FETCH
 
 extern "C" void qsa_retention_state_launch(
     const bf16_t* x, long long xstride, long long voff, const bf16_t* planes,
