@@ -262,7 +262,8 @@ def bench_models(layers: int = 8) -> None:
                 prompts = [[(i * 7 + j) % 30_000 for j in range(2048)]
                            for i in range(B)]
                 seqs = [eng.submit(p, 260) for p in prompts]
-                eng._admit()
+                while eng.pending:
+                    eng._admit()
                 eng._decode_run_graph(seqs, 2)        # capture and warm up
                 torch.cuda.synchronize()
                 t = time.perf_counter()

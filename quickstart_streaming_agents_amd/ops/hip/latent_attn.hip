@@ -45,60 +45,83 @@ qsa_head_matmul(const T* __restrict__ x, long long xrow,
   }
 }
 
-// Matrix cores: wave = 16 rows x 64 columns; W rows are the A operand, so a
-// lane ends up with 4 consecutive columns of one row.
+// Matrix cores.  A wave computes 16 columns of one head for up to 64 rows; W
+// rows are the A operand, so a lane ends up with 4 consecutive columns of one
+// row.  SPLIT: the four waves of a block share the columns, split K (every
+// load of the product is in flight at once) and meet in LDS; otherwise they
+// take 16 columns each.
+template <bool SPLIT>
 __global__ void __launch_bounds__(256)
 qsa_head_matmul_mfma(const bf16_t* __restrict__ x, long long xrow,
                      const bf16_t* __restrict__ W,
                      const bf16_t* __restrict__ gate, long long grow,
                      bf16_t* __restrict__ out, int M, int H, int N, int K,
-                     int NG) {
-  const int lane = threadIdx.x & 63;
+                     int NT) {
+  __shared__ f32x4_v red[SPLIT ? 4 : 1][4][64];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int col = lane & 15, hi = lane >> 4;
-  const int ng = blockIdx.x % NG;
-  const int h = (blockIdx.x / NG) % H;
-  const int mt = (blockIdx.x / (NG * H)) * 4 + (threadIdx.x >> 6);
-  if (mt * 16 >= M) return;                 // whole waves, no barrier below
-  const int m = mt * 16 + col;
-  const bf16_t* xr = x + (long long)min(m, M - 1) * xrow + (long long)h * K;
-  const bf16_t* wr[4];
+  const int nt = SPLIT ? blockIdx.x % NT : blockIdx.x % NT * 4 + wave;
+  const int h = (blockIdx.x / NT) % H;
+  const int m0 = (blockIdx.x / (NT * H)) * 64;
+  const int nmt = min(4, (M - m0 + 15) / 16);
+  const bf16_t* xr[4];
 #pragma unroll
   for (int t = 0; t < 4; ++t)
-    wr[t] = W + ((long long)h * N + min(ng * 64 + t * 16 + col, N - 1)) * K;
+    xr[t] = x + (long long)min(m0 + t * 16 + col, M - 1) * xrow +
+            (long long)h * K;
+  const bf16_t* wr = W + ((long long)h * N + min(nt * 16 + col, N - 1)) * K;
   const bf16x8_v zero = {0, 0, 0, 0, 0, 0, 0, 0};
   f32x4_v acc[4];
 #pragma unroll
   for (int t = 0; t < 4; ++t) acc[t] = (f32x4_v){0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
-  for (int k0 = 0; k0 < K; k0 += 32) {
-    const int k = k0 + hi * 8;
-    const bool ok = k < K;                  // K % 8 == 0
-    const int kk = ok ? k : 0;
-    bf16x8_v b = *reinterpret_cast<const bf16x8_v*>(xr + kk);
-    b = ok ? b : zero;
+  const int per = SPLIT ? ((K + 31) / 32 + 3) / 4 * 32 : K;
+  const int ka = SPLIT ? wave * per : 0;
+  const int k1 = min(K, ka + per);
+  for (int k0 = ka; k0 < k1; k0 += 128) {
+    bf16x8_v a[4];
 #pragma unroll
-    for (int t = 0; t < 4; ++t) {
-      bf16x8_v a = *reinterpret_cast<const bf16x8_v*>(wr[t] + kk);
-      a = ok ? a : zero;
-      acc[t] = mfma_bf16(a, b, acc[t]);
+    for (int s = 0; s < 4; ++s) {
+      const int k = k0 + s * 32 + hi * 8;           // K % 8 == 0
+      const bf16x8_v v = *reinterpret_cast<const bf16x8_v*>(
+          wr + (k < k1 ? k : 0));
+      a[s] = k < k1 ? v : zero;
     }
-  }
-  if (m < M) {
 #pragma unroll
     for (int t = 0; t < 4; ++t) {
-      const int n0 = ng * 64 + t * 16 + hi * 4;
-      if (n0 < N) {                         // N % 4 == 0
-        float v[4] = {acc[t][0], acc[t][1], acc[t][2], acc[t][3]};
-        if (gate) {
-          float g[4];
-          ldv<bf16_t, 4>(gate + (long long)m * grow + (long long)h * N + n0,
-                         g);
+      if (t >= nmt) break;                          // uniform
 #pragma unroll
-          for (int r = 0; r < 4; ++r) v[r] /= 1.f + __expf(-g[r]);
-        }
-        stv<bf16_t, 4>(out + ((long long)m * H + h) * N + n0, v);
+      for (int s = 0; s < 4; ++s) {
+        const int k = k0 + s * 32 + hi * 8;
+        bf16x8_v b = *reinterpret_cast<const bf16x8_v*>(
+            xr[t] + (k < k1 ? k : 0));
+        b = k < k1 ? b : zero;
+        acc[t] = mfma_bf16(a[s], b, acc[t]);
       }
     }
+  }
+  const int n0 = nt * 16 + hi * 4;
+  auto finish = [&](int m, f32x4_v s) {
+    if (m >= M || n0 >= N) return;                  // N % 4 == 0
+    float v[4] = {s[0], s[1], s[2], s[3]};
+    if (gate) {
+      float g[4];
+      ldv<bf16_t, 4>(gate + (long long)m * grow + (long long)h * N + n0, g);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) v[r] /= 1.f + __expf(-g[r]);
+    }
+    stv<bf16_t, 4>(out + ((long long)m * H + h) * N + n0, v);
+  };
+  if (SPLIT) {
+#pragma unroll
+    for (int t = 0; t < 4; ++t) red[wave][t][lane] = acc[t];
+    lds_barrier();
+    finish(m0 + wave * 16 + col,
+           (red[0][wave][lane] + red[1 % (SPLIT ? 4 : 1)][wave][lane]) +
+               (red[2 % (SPLIT ? 4 : 1)][wave][lane] +
+                red[3 % (SPLIT ? 4 : 1)][wave][lane]));
+  } else {
+#pragma unroll
+    for (int t = 0; t < 4; ++t) finish(m0 + t * 16 + col, acc[t]);
   }
 }
 
@@ -108,12 +131,15 @@ extern "C" void qsa_head_matmul_launch(const void* x, long long xrow,
                                        int H, int N, int K, int f32,
                                        int mfma, hipStream_t st) {
   if (mfma) {
-    const int NG = (N + 63) / 64;
-    dim3 grid((unsigned)((M + 63) / 64 * H * NG));
-    hipLaunchKernelGGL(qsa_head_matmul_mfma, grid, dim3(256), 0, st,
+    const bool split = K > 128;
+    const int NT = split ? (N + 15) / 16 : (N + 63) / 64;
+    dim3 grid((unsigned)((M + 63) / 64 * H * NT));
+    auto* kernel = split ? qsa_head_matmul_mfma<true>
+                         : qsa_head_matmul_mfma<false>;
+    hipLaunchKernelGGL(kernel, grid, dim3(256), 0, st,
                        (const bf16_t*)x, xrow, (const bf16_t*)W,
                        (const bf16_t*)gate, grow, (bf16_t*)out, M, H, N, K,
-                       NG);
+                       NT);
     return;
   }
   dim3 grid((unsigned)((long long)M * H));
@@ -226,7 +252,7 @@ extern "C" void qsa_latent_rows_launch(
 // splits meet in qsa_latent_merge, which also adds the sink.
 // ---------------------------------------------------------------------------
 template <int DTW>  // latent columns <= 64 * DTW
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, 2)
 qsa_latent_rows_mfma(const bf16_t* __restrict__ qa,
                      const bf16_t* __restrict__ cache,
                      const int* __restrict__ block_table, int max_pages,
@@ -283,20 +309,20 @@ qsa_latent_rows_mfma(const bf16_t* __restrict__ qa,
         const int r = g / (DP / 8), c = (g % (DP / 8)) * 8;
         const bool ok = c < KR && r >= a && r < b;
         const uint4 v = *reinterpret_cast<const uint4*>(
-            base + (ok ? (long long)r * KR + c : 0));
+            base + (unsigned)(ok ? r * KR + c : 0));
         reg[u] = ok ? v : make_uint4(0, 0, 0, 0);
       }
     };
     fetch(pa);
     for (int pg = pa; pg < pb; ++pg) {
-      __syncthreads();                              // readers of ct/ps done
+      lds_barrier();                              // readers of ct/ps done
 #pragma unroll
       for (int u = 0; u < LD; ++u) {
         const int g = tid + u * 256;
         const int r = g / (DP / 8), c = (g % (DP / 8)) * 8;
         *reinterpret_cast<uint4*>(&ct[r * CP + c]) = reg[u];
       }
-      __syncthreads();
+      lds_barrier();
       if (pg + 1 < pb) fetch(pg + 1);
       f32x4_v s4 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -315,7 +341,7 @@ qsa_latent_rows_mfma(const bf16_t* __restrict__ qa,
       mx = fmaxf(mx, __shfl_xor(mx, 16, QSA_WAVE));
       mx = fmaxf(mx, __shfl_xor(mx, 32, QSA_WAVE));
       if (hi == 0) smax[wave][col] = mx;
-      __syncthreads();
+      lds_barrier();
       float mn = m;
 #pragma unroll
       for (int w = 0; w < 4; ++w) mn = fmaxf(mn, smax[w][col]);
@@ -330,7 +356,7 @@ qsa_latent_rows_mfma(const bf16_t* __restrict__ qa,
           make_uint2(cvt_bf16x2(p[0], p[1]), cvt_bf16x2(p[2], p[3]));
 #pragma unroll
       for (int t = 0; t < DTW; ++t) acc[t] *= alpha;
-      __syncthreads();
+      lds_barrier();
 #pragma unroll
       for (int s = 0; s < 2; ++s) {
         const uint2 x0 = ps[s * 2][lane], x1 = ps[s * 2 + 1][lane];
@@ -348,9 +374,9 @@ qsa_latent_rows_mfma(const bf16_t* __restrict__ qa,
   // l: sum over the hi groups of each wave, then over the waves
   l += __shfl_xor(l, 16, QSA_WAVE);
   l += __shfl_xor(l, 32, QSA_WAVE);
-  __syncthreads();
+  lds_barrier();
   if (hi == 0) smax[wave][col] = l;
-  __syncthreads();
+  lds_barrier();
   if (head < H) {
     const long long o = (row * H + head) * NS + split;
     if (wave == 0 && hi == 0) {
@@ -375,29 +401,31 @@ qsa_latent_merge(const float* __restrict__ part_o,
                  const float* __restrict__ part_ml,
                  const bf16_t* __restrict__ sink, bf16_t* __restrict__ out,
                  int H, int KR, int NS) {
+  extern __shared__ float ws[];                     // NS weights
   const long long rh = blockIdx.x;
   const float* ml = part_ml + rh * NS * 2;
   const float sk = bf16_to_f32(sink[rh % H]) * LOG2E;
-  float top = sk;
-  for (int s = 0; s < NS; ++s)
+  const int lane = threadIdx.x & 63;
+  float top = NEG_BIG;
+  for (int s = lane; s < NS; s += 64)
     if (ml[2 * s + 1] > 0.f) top = fmaxf(top, ml[2 * s]);
-  float den = exp2f(sk - top);
-  for (int s = 0; s < NS; ++s)
-    if (ml[2 * s + 1] > 0.f) den = fmaf(exp2f(ml[2 * s] - top), ml[2 * s + 1], den);
-  const float inv = 1.f / den;
+  top = fmaxf(wave_reduce_max(top), sk);
+  float den = 0.f;
+  for (int s = lane; s < NS; s += 64) {
+    const float w = ml[2 * s + 1] > 0.f ? exp2f(ml[2 * s] - top) : 0.f;
+    if (threadIdx.x < 64) ws[s] = w;
+    den = fmaf(w, ml[2 * s + 1], den);
+  }
+  const float inv = 1.f / (wave_reduce_sum(den) + exp2f(sk - top));
+  __syncthreads();
   for (int k = threadIdx.x * 4; k < KR; k += blockDim.x * 4) {
-    float a[4] = {0.f, 0.f, 0.f, 0.f};
-    for (int s = 0; s < NS; ++s) {
-      if (ml[2 * s + 1] <= 0.f) continue;
-      const float w = exp2f(ml[2 * s] - top);
-      const float4 p =
-          *reinterpret_cast<const float4*>(part_o + (rh * NS + s) * KR + k);
-      a[0] = fmaf(w, p.x, a[0]); a[1] = fmaf(w, p.y, a[1]);
-      a[2] = fmaf(w, p.z, a[2]); a[3] = fmaf(w, p.w, a[3]);
-    }
-#pragma unroll
-    for (int j = 0; j < 4; ++j) a[j] *= inv;
-    stv<bf16_t, 4>(out + rh * KR + k, a);
+    f32x4_v a = {0.f, 0.f, 0.f, 0.f};
+    const float* po = part_o + rh * NS * KR + k;
+#pragma unroll 8
+    for (int s = 0; s < NS; ++s)
+      a += ws[s] * *reinterpret_cast<const f32x4_v*>(po + (long long)s * KR);
+    float v[4] = {a[0] * inv, a[1] * inv, a[2] * inv, a[3] * inv};
+    stv<bf16_t, 4>(out + rh * KR + k, v);
   }
 }
 
@@ -419,7 +447,8 @@ extern "C" void qsa_latent_rows_mfma_launch(
 #undef QSA_LR
   const int th = KR >= 1024 ? 256 : (KR / 4 + 63) / 64 * 64;
   hipLaunchKernelGGL(qsa_latent_merge, dim3((unsigned)((long long)R * H)),
-                     dim3(th), 0, st, part_o, part_ml, sink, out, H, KR, NS);
+                     dim3(th), sizeof(float) * NS, st, part_o, part_ml, sink,
+                     out, H, KR, NS);
 }
 
 // ---------------------------------------------------------------------------
@@ -434,7 +463,7 @@ extern "C" void qsa_latent_rows_mfma_launch(
 //   begin at ctx_off and hold positions ctx_pos..start+len-1.
 // ---------------------------------------------------------------------------
 template <int KS, int ET>  // D <= 32*KS, E <= 16*ET
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, ET <= 8 ? 2 : 1)
 qsa_window_attn_prefill(const bf16_t* __restrict__ q, long long qstride,
                         const bf16_t* __restrict__ kv, long long kvstride,
                         const bf16_t* __restrict__ gate, long long gstride,
@@ -512,7 +541,7 @@ qsa_window_attn_prefill(const bf16_t* __restrict__ q, long long qstride,
   };
   fetch(first);
   for (int pos = first; pos <= last; pos += 64) {
-    __syncthreads();
+    lds_barrier();
 #pragma unroll
     for (int u = 0; u < KL; ++u) {
       const int g = tid + u * 256;
@@ -524,7 +553,7 @@ qsa_window_attn_prefill(const bf16_t* __restrict__ q, long long qstride,
       if (g < 64 * VG)
         *reinterpret_cast<uint4*>(&vt[(g / VG) * VP + (g % VG) * 8]) = vr[u];
     }
-    __syncthreads();
+    lds_barrier();
     if (pos + 64 <= last) fetch(pos + 64);
     if (pos > wlast || pos + 63 < wfirst) continue;   // nothing for this wave
     f32x4_v s4[4];

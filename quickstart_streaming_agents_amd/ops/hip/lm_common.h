@@ -99,6 +99,14 @@ __device__ __forceinline__ void split4_bf16(float a, float b, float c, float d,
                   cvt_bf16x2(c - h1.x, d - h1.y));
 }
 
+// Barrier that orders LDS accesses only: global loads and stores in flight
+// stay in flight (their users wait for the registers).
+__device__ __forceinline__ void lds_barrier() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
+  __builtin_amdgcn_s_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
+}
+
 // Transposing LDS read: within 16 lanes, lane i supplies the address of 4
 // consecutive elements of row i/4, columns (i%4)*4.. of a 4 x 16 block and
 // receives column i, i.e. 4 consecutive rows of one column.

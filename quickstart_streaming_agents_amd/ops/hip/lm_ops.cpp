@@ -62,11 +62,11 @@ extern "C" void qsa_retention_rotate_launch(const bf16_t*, long long,
     int, int, float, int, hipStream_t);
 extern "C" void qsa_retention_state_launch(const bf16_t*, long long,
     long long, const bf16_t*, long long, const float*, float*, const int*,
-    const int*, const int*, const int*, const int*, bf16_t*, long long, int,
-    int, int, int, int, int, hipStream_t);
+    const int*, const int*, const int*, const int*, void*, int, int, int,
+    int, int, int, hipStream_t);
 extern "C" void qsa_retention_out_launch(const bf16_t*, long long, long long,
     const bf16_t*, long long, const float*, const int*, const int*,
-    const int*, const int*, const int*, const bf16_t*, long long, bf16_t*,
+    const int*, const int*, const int*, const void*, long long, bf16_t*,
     int, int, int, int, float, hipStream_t);
 extern "C" void qsa_head_matmul_launch(const void*, long long, const void*,
     const void*, long long, void*, int, int, int, int, int, int, hipStream_t);
@@ -222,7 +222,7 @@ Tensor retention_decode(Tensor x, Tensor cos_t, Tensor sin_t, Tensor decay,
   CHK_I32(slots); CHK_I32(seq_lens);
   const int B = (int)x.size(0);
   TORCH_CHECK(slots.numel() == B && seq_lens.numel() == B, "slots/seq_lens");
-  TORCH_CHECK(2 * r.D + 2 * r.E <= 12000, "head too wide for the decode block");
+  TORCH_CHECK(2 * r.D + 2 * r.E <= 8000, "head too wide for the decode block");
   auto out = torch::empty({B, (long long)r.H * r.E}, x.options());
   if (B == 0) return out;
   const int v4 = r.E % 4 == 0 && (2LL * r.H * r.D) % 4 == 0 &&
@@ -297,8 +297,8 @@ void retention_chunked(Tensor x, Tensor cos_t, Tensor sin_t,
   TORCH_CHECK(out.size(0) == T && out.size(1) == (long long)r.H * r.E, "out");
   if (n == 0 || nc == 0) return;
   const int DP = pad_dim(r.D), EP = (r.E + 15) / 16 * 16;
-  auto planes = torch::empty({4, T, r.H, DP}, x.options());
-  auto prefix = torch::empty({2, nc, r.H, EP, DP}, x.options());
+  auto planes = torch::empty({3, T, r.H, DP}, x.options());
+  auto prefix = torch::empty({nc, r.H, 2, EP, DP}, x.options());
   hipStream_t st = cur_stream();
   const long long voff = 2LL * r.H * r.D;
   qsa_retention_rotate_launch(u16(x), x.stride(0), cos_t.data_ptr<float>(),
@@ -310,12 +310,12 @@ void retention_chunked(Tensor x, Tensor cos_t, Tensor sin_t,
                              state.data_ptr<float>(), slots.data_ptr<int>(),
                              off.data_ptr<int>(), start.data_ptr<int>(),
                              len.data_ptr<int>(), chunk0.data_ptr<int>(),
-                             u16m(prefix), nc, n, r.H, r.D, DP, r.E, EP, st);
+                             prefix.data_ptr(), n, r.H, r.D, DP, r.E, EP, st);
   qsa_retention_out_launch(u16(x), x.stride(0), voff, u16(planes), T,
                            log2_decay.data_ptr<float>(), off.data_ptr<int>(),
                            start.data_ptr<int>(), len.data_ptr<int>(),
                            chunk_item.data_ptr<int>(),
-                           chunk_t0.data_ptr<int>(), u16(prefix), nc,
+                           chunk_t0.data_ptr<int>(), prefix.data_ptr(), nc,
                            u16m(out), r.H, DP, r.E, EP, (float)eps, st);
 }
 
@@ -377,8 +377,12 @@ Tensor latent_rows(Tensor qa, Tensor cache, Tensor block_table,
     const int HT = (H + 15) / 16;
     int pages = mp;
     if (window > 0) pages = (int)std::min<long>(mp, (window + 62) / 64 + 1);
-    long long ns = (1024 + (long long)R * HT - 1) / ((long long)R * HT);
+    // two blocks fit a CU: enough of them to fill the chip once, and no
+    // shares that differ by a page when they need not
+    long long ns = (512 + (long long)R * HT - 1) / ((long long)R * HT);
     ns = std::max<long long>(1, std::min<long long>(ns, pages));
+    const long long per = (pages + ns - 1) / ns;
+    ns = (pages + per - 1) / per;
     auto of = qa.options().dtype(at::kFloat);
     auto po = torch::empty({R, H, ns, KR}, of);
     auto pm = torch::empty({R, H, ns, 2}, of);

@@ -15,14 +15,16 @@
 //   qsa_retention_seq      token loop per (portion, head), any size and
 //                          storage type; the f32 path.
 //   chunked prefill (bf16 storage, matrix cores), chunks of 64 tokens:
-//     qsa_retention_rotate   rotated q, k as bf16 hi/lo planes, zero-padded
+//     qsa_retention_rotate   rotated q (bf16) and k (bf16 hi/lo), padded
 //     qsa_retention_state    walks the chunks of a portion, state tile in
 //                            accumulators; leaves the state before each
-//                            chunk as hi/lo planes [chunk, H, vdim, dim]
+//                            chunk as hi/lo matrix-core operands
 //     qsa_retention_out      per (chunk, head): inter-chunk read-out,
 //                            intra-chunk masked product, norm, gate
-// Every operand that f32 rounding matters for is a hi/lo pair, so the
-// chunked result agrees with the token loop to ~2^-16; v is bf16 already.
+// Everything that enters the recurrence is a bf16 hi/lo pair on the matrix
+// cores (k, the decayed v, the state, the intra-chunk weights), so the chunked
+// recurrence agrees with the token loop to ~2^-16; q, which only reads the
+// state out, is rounded once like any activation, and v is bf16 already.
 #include "lm_common.h"
 
 #define RC 64  // tokens per chunk
@@ -45,7 +47,7 @@ __device__ __forceinline__ float rot_elem(const T* x, int d, int rot,
 // Decode: one block per (row, head).
 // ---------------------------------------------------------------------------
 template <typename T, int VEC>
-__global__ void __launch_bounds__(512)
+__global__ void __launch_bounds__(1024)
 qsa_retention_decode(const T* __restrict__ x, long long xstride,
                      const float* __restrict__ cos_t,
                      const float* __restrict__ sin_t,
@@ -59,7 +61,7 @@ qsa_retention_decode(const T* __restrict__ x, long long xstride,
   float* ks = qs + D;             // D
   float* os = ks + D;             // E
   float* red = os + (E + 3) / 4 * 4;  // threads * VEC
-  __shared__ float scratch[8];
+  __shared__ float scratch[16];
   const int b = blockIdx.x / H, h = blockIdx.x % H;
   const int tid = threadIdx.x, nth = blockDim.x;
   const int pos = seq_lens[b] - 1;
@@ -143,7 +145,9 @@ extern "C" void qsa_retention_decode_launch(
   const int nv = vec4 ? E / 4 : E;
   int cw = 1;
   while (cw < nv && cw < 256) cw <<= 1;
-  const int threads = 256;
+  // few blocks: wide ones, so that enough of the state is in flight
+  const int threads =
+      (long long)B * H <= 512 && (long long)D * E >= 16384 ? 1024 : 256;
   const size_t lds = sizeof(float) *
       (2 * (size_t)D + (E + 3) / 4 * 4 + threads * (vec4 ? 4 : 1));
 #define QSA_RD(T, V)                                                         \
@@ -246,8 +250,11 @@ extern "C" void qsa_retention_seq_launch(
 }
 
 // ---------------------------------------------------------------------------
-// Chunked prefill, step 1: planes[p][row][h][DP], p = q.hi, q.lo, k.hi, k.lo
+// Chunked prefill, step 1: planes[p][row][h][DP], p = q, k.hi, k.lo
 // ---------------------------------------------------------------------------
+// One thread per 8 dims of a head of a row, q and k.  FAST: whole groups on
+// either side of the rotation pairs (rot % 16 == 0, D % 8 == 0, 16 B rows).
+template <bool FAST>
 __global__ void __launch_bounds__(256)
 qsa_retention_rotate(const bf16_t* __restrict__ x, long long xstride,
                      const float* __restrict__ cos_t,
@@ -256,34 +263,61 @@ qsa_retention_rotate(const bf16_t* __restrict__ x, long long xstride,
                      bf16_t* __restrict__ planes, long long rows, int H,
                      int D, int DP, int rot, float kscale, int table_len) {
   const long long plane = rows * H * DP;
-  const long long n = rows * H * (DP / 4);
-  for (long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x; i < n;
-       i += (long long)gridDim.x * blockDim.x) {
-    const int d0 = (int)(i % (DP / 4)) * 4;
-    const long long rh = i / (DP / 4);
-    const int h = (int)(rh % H);
-    const long long row = rh / H;
-    int p = positions[row];
-    p = p < table_len ? p : table_len - 1;
-    const float* cs = cos_t + (long long)p * (rot >> 1);
-    const float* sn = sin_t + (long long)p * (rot >> 1);
+  const int per_row = H * (DP / 8);
+  const long long row = blockIdx.x;
+  const int half = rot >> 1;
+  int p = positions[row];
+  p = p < table_len ? p : table_len - 1;
+  const float* cs = cos_t + (long long)p * half;
+  const float* sn = sin_t + (long long)p * half;
+  for (int g = threadIdx.x; g < per_row; g += blockDim.x) {
+    const int h = g / (DP / 8), d0 = (g % (DP / 8)) * 8;
     const bf16_t* q = x + row * xstride + (long long)h * D;
     const bf16_t* k = q + (long long)H * D;
-    float qv[4], kv[4];
+    float qv[8], kv[8];
+    if (FAST) {
+      if (d0 < D) {
+        ldv<bf16_t, 8>(q + d0, qv);
+        ldv<bf16_t, 8>(k + d0, kv);
+        if (d0 < rot) {
+          const bool lo = d0 < half;
+          const int o = lo ? d0 + half : d0 - half, c = lo ? d0 : d0 - half;
+          float qo[8], ko[8], cc[8], ss[8];
+          ldv<bf16_t, 8>(q + o, qo);
+          ldv<bf16_t, 8>(k + o, ko);
+          ldv<float, 8>(cs + c, cc);
+          ldv<float, 8>(sn + c, ss);
+          const float sg = lo ? -1.f : 1.f;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const int d = d0 + j;
-      qv[j] = d < D ? rot_elem<bf16_t>(q, d, rot, cs, sn) : 0.f;
-      kv[j] = d < D ? rot_elem<bf16_t>(k, d, rot, cs, sn) * kscale : 0.f;
+          for (int j = 0; j < 8; ++j) {
+            qv[j] = qv[j] * cc[j] + sg * qo[j] * ss[j];
+            kv[j] = kv[j] * cc[j] + sg * ko[j] * ss[j];
+          }
+        }
+      } else {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) qv[j] = kv[j] = 0.f;
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        const int d = d0 + j;
+        qv[j] = d < D ? rot_elem<bf16_t>(q, d, rot, cs, sn) : 0.f;
+        kv[j] = d < D ? rot_elem<bf16_t>(k, d, rot, cs, sn) : 0.f;
+      }
     }
-    uint2 a, b;
-    bf16_t* o = planes + rh * DP + d0;
-    split4_bf16(qv[0], qv[1], qv[2], qv[3], a, b);
-    *reinterpret_cast<uint2*>(o) = a;
-    *reinterpret_cast<uint2*>(o + plane) = b;
-    split4_bf16(kv[0], kv[1], kv[2], kv[3], a, b);
-    *reinterpret_cast<uint2*>(o + 2 * plane) = a;
-    *reinterpret_cast<uint2*>(o + 3 * plane) = b;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) kv[j] *= kscale;
+    uint2 a0, b0, a1, b1;
+    bf16_t* o = planes + (row * H + h) * DP + d0;
+    *reinterpret_cast<uint4*>(o) =
+        make_uint4(cvt_bf16x2(qv[0], qv[1]), cvt_bf16x2(qv[2], qv[3]),
+                   cvt_bf16x2(qv[4], qv[5]), cvt_bf16x2(qv[6], qv[7]));
+    split4_bf16(kv[0], kv[1], kv[2], kv[3], a0, b0);
+    split4_bf16(kv[4], kv[5], kv[6], kv[7], a1, b1);
+    *reinterpret_cast<uint4*>(o + plane) = make_uint4(a0.x, a0.y, a1.x, a1.y);
+    *reinterpret_cast<uint4*>(o + 2 * plane) =
+        make_uint4(b0.x, b0.y, b1.x, b1.y);
   }
 }
 
@@ -292,21 +326,30 @@ extern "C" void qsa_retention_rotate_launch(
     const float* sin_t, const int* positions, bf16_t* planes, long long rows,
     int H, int D, int DP, int rot, float kscale, int table_len,
     hipStream_t st) {
-  const long long n = rows * H * (DP / 4);
-  const long long want = (n + 255) / 256;
-  hipLaunchKernelGGL(qsa_retention_rotate,
-                     dim3((unsigned)(want > 32768 ? 32768 : want)), dim3(256),
-                     0, st, x, xstride, cos_t, sin_t, positions, planes, rows,
-                     H, D, DP, rot, kscale, table_len);
+  // x rows are 16 B aligned and H*D % 4 == 0 on this path
+  const bool fast = rot % 16 == 0 && D % 8 == 0;
+  int threads = (H * (DP / 8) + 63) / 64 * 64;
+  threads = threads > 256 ? 256 : threads;
+#define QSA_RR(F)                                                          \
+  hipLaunchKernelGGL((qsa_retention_rotate<F>), dim3((unsigned)rows),      \
+                     dim3(threads), 0, st, x, xstride, cos_t, sin_t,       \
+                     positions, planes, rows, H, D, DP, rot, kscale,       \
+                     table_len)
+  if (fast) QSA_RR(true); else QSA_RR(false);
+#undef QSA_RR
 }
 
 // ---------------------------------------------------------------------------
-// Step 2: state walk.  Block = (portion, head, 64 value columns); wave w owns
-// 16 of the columns and all DP rows of the state tile in accumulators.
+// Step 2: state walk.  Block = (portion, head, 64 value columns); a wave owns
+// 16 of the columns and 1/DH of the state rows in accumulators.
 //   S_(c+1) = decay^n S_c + sum_j k_j (decay^(n-1-j) v_j)^T
+// The state before a chunk is left in the operand order of step 3: for value
+// tile vt and 32 dims ks, 16 B per lane (column vt*16 + lane%16; dims
+// ks*32 + hi*4 .. +3 and ks*32 + 16 + hi*4 .. +3), so both sides move whole
+// 1 KiB lines:  prefix[chunk][head][plane][vt][ks][lane][8]
 // ---------------------------------------------------------------------------
-template <int KS>  // DP = 32 * KS
-__global__ void __launch_bounds__(256)
+template <int KS, int DH>  // DP = 32 * KS, 4 * DH waves
+__global__ void __launch_bounds__(256 * DH)
 qsa_retention_state(const bf16_t* __restrict__ x, long long xstride,
                     long long voff, const bf16_t* __restrict__ planes,
                     long long rows, const float* __restrict__ log2_decay,
@@ -314,19 +357,23 @@ qsa_retention_state(const bf16_t* __restrict__ x, long long xstride,
                     const int* __restrict__ off, const int* __restrict__ start,
                     const int* __restrict__ len,
                     const int* __restrict__ chunk0,
-                    bf16_t* __restrict__ prefix, long long n_chunks, int H,
-                    int D, int E, int EP) {
+                    u32x4_v* __restrict__ prefix, int H, int D, int E,
+                    int EP) {
   constexpr int DP = 32 * KS;
   constexpr int KP = DP + 16;       // LDS pitches (elements)
   constexpr int VP = 64 + 16;
-  constexpr int KLD = RC * DP / 8 / 256;   // 16 B groups per thread and plane
+  constexpr int NTH = 256 * DH;
+  constexpr int KLD = RC * DP / 8 * 2 / NTH;  // 16 B groups of k per thread
+  constexpr int VLD = RC * 8 / NTH;           // ... and of v
+  constexpr int NT_ = 2 * KS / DH;            // 16-row tiles per wave
   __shared__ __attribute__((aligned(16))) bf16_t kt[2][RC * KP];
   __shared__ __attribute__((aligned(16))) bf16_t vt[2][RC * VP];
   const int VT = (EP + 63) / 64;
   const int vtile = blockIdx.x % VT;
   const int h = (blockIdx.x / VT) % H;
   const int it = blockIdx.x / (VT * H);
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int tid = threadIdx.x, lane = tid & 63, wave = (tid >> 6) & 3;
+  const int tile0 = (tid >> 8) * NT_;          // this wave's first row tile
   const int col = lane & 15, hi = lane >> 4;
   const int n = len[it], p0 = start[it], r0 = off[it], slot = slots[it];
   const float l2d = log2_decay[h];
@@ -334,33 +381,32 @@ qsa_retention_state(const bf16_t* __restrict__ x, long long xstride,
   const int e = v0 + wave * 16 + col;          // this lane's value column
   float* S = state + ((long long)slot * H + h) * D * E;
   const long long plane = rows * H * DP;
-  const bf16_t* kpl = planes + 2 * plane;
+  const bf16_t* kpl = planes + plane;
 
-  f32x4_v acc[2 * KS];
+  f32x4_v acc[NT_];
 #pragma unroll
-  for (int t = 0; t < 2 * KS; ++t)
+  for (int t = 0; t < NT_; ++t)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int d = t * 16 + hi * 4 + r;
+      const int d = (tile0 + t) * 16 + hi * 4 + r;
       acc[t][r] = (p0 > 0 && d < D && e < E) ? S[(long long)d * E + e] : 0.f;
     }
 
-  u32x4_v kh[KLD], kl[KLD], vreg[2];
+  u32x4_v kreg[KLD], vreg[VLD];
 #define QSA_FETCH(t0_)                                                        \
   {                                                                           \
     _Pragma("unroll") for (int u = 0; u < KLD; ++u) {                         \
-      const int g = tid + u * 256;                                            \
-      const int tr = min((t0_) + g / (DP / 8), n - 1);                        \
-      const bf16_t* src = kpl + ((long long)(r0 + tr) * H + h) * DP +         \
-                          (g % (DP / 8)) * 8;                                 \
-      kh[u] = *reinterpret_cast<const u32x4_v*>(src);                           \
-      kl[u] = *reinterpret_cast<const u32x4_v*>(src + plane);                   \
+      const int g = tid + u * NTH; /* plane, row, group */                    \
+      const int tr = min((t0_) + g / (DP / 8) % RC, n - 1);                   \
+      kreg[u] = *reinterpret_cast<const u32x4_v*>(                            \
+          kpl + (g / (RC * DP / 8)) * plane +                                 \
+          ((long long)(r0 + tr) * H + h) * DP + (g % (DP / 8)) * 8);          \
     }                                                                         \
-    _Pragma("unroll") for (int u = 0; u < 2; ++u) {                           \
-      const int g = tid + u * 256;                                            \
+    _Pragma("unroll") for (int u = 0; u < VLD; ++u) {                         \
+      const int g = tid + u * NTH;                                            \
       const int tr = min((t0_) + (g >> 3), n - 1);                            \
       const int cc = min(v0 + (g & 7) * 8, E - 8); /* E % 8 == 0 */           \
-      vreg[u] = *reinterpret_cast<const u32x4_v*>(                              \
+      vreg[u] = *reinterpret_cast<const u32x4_v*>(                            \
           x + (long long)(r0 + tr) * xstride + voff + (long long)h * E + cc); \
     }                                                                         \
   }
@@ -369,17 +415,17 @@ qsa_retention_state(const bf16_t* __restrict__ x, long long xstride,
   for (int c = 0; c < nc; ++c) {
     const int t0 = c * RC;
     const int m = min(RC, n - t0);
-    __syncthreads();                 // previous chunk's LDS readers are done
+    lds_barrier();                   // previous chunk's LDS readers are done
 #pragma unroll
     for (int u = 0; u < KLD; ++u) {
-      const int g = tid + u * 256;
-      const int o = g / (DP / 8) * KP + (g % (DP / 8)) * 8;
-      *reinterpret_cast<u32x4_v*>(&kt[0][o]) = kh[u];
-      *reinterpret_cast<u32x4_v*>(&kt[1][o]) = kl[u];
+      const int g = tid + u * NTH;
+      *reinterpret_cast<u32x4_v*>(
+          &kt[g / (RC * DP / 8)][g / (DP / 8) % RC * KP +
+                                 (g % (DP / 8)) * 8]) = kreg[u];
     }
 #pragma unroll
-    for (int u = 0; u < 2; ++u) {
-      const int g = tid + u * 256;
+    for (int u = 0; u < VLD; ++u) {
+      const int g = tid + u * NTH;
       const int row = g >> 3, cc = (g & 7) * 8;
       const bool ok = row < m && v0 + cc < E;
       const float f = exp2f((float)(m - 1 - row) * l2d);
@@ -395,26 +441,30 @@ qsa_retention_state(const bf16_t* __restrict__ x, long long xstride,
       *reinterpret_cast<uint4*>(&vt[1][row * VP + cc]) =
           make_uint4(l0.x, l0.y, l1.x, l1.y);
     }
-    __syncthreads();
+    lds_barrier();
     if (c + 1 < nc) QSA_FETCH(t0 + RC)
 
     // state before this chunk (nothing precedes the first token)
-    if ((c > 0 || p0 > 0) && e < EP) {
-      bf16_t* ph = prefix +
-          (((long long)(chunk0[it] + c) * H + h) * EP + e) * DP;
-      bf16_t* pl = ph + n_chunks * H * EP * DP;
+    if ((c > 0 || p0 > 0) && v0 + wave * 16 < EP) {
+      const int NT = EP / 16, vt16 = v0 / 16 + wave;
+      u32x4_v* ph = prefix +
+          ((((long long)(chunk0[it] + c) * H + h) * 2) * NT + vt16) * KS * 64 +
+          lane;
+      u32x4_v* pl = ph + (long long)NT * KS * 64;
 #pragma unroll
-      for (int t = 0; t < 2 * KS; ++t) {
-        uint2 a, b;
-        split4_bf16(acc[t][0], acc[t][1], acc[t][2], acc[t][3], a, b);
-        const int d = t * 16 + hi * 4;
-        *reinterpret_cast<uint2*>(ph + d) = a;
-        *reinterpret_cast<uint2*>(pl + d) = b;
+      for (int s = 0; s < NT_ / 2; ++s) {
+        uint2 a0, b0, a1, b1;
+        split4_bf16(acc[2 * s][0], acc[2 * s][1], acc[2 * s][2],
+                    acc[2 * s][3], a0, b0);
+        split4_bf16(acc[2 * s + 1][0], acc[2 * s + 1][1], acc[2 * s + 1][2],
+                    acc[2 * s + 1][3], a1, b1);
+        ph[(tile0 / 2 + s) * 64] = (u32x4_v){a0.x, a0.y, a1.x, a1.y};
+        pl[(tile0 / 2 + s) * 64] = (u32x4_v){b0.x, b0.y, b1.x, b1.y};
       }
     }
     const float dn = exp2f((float)m * l2d);
 #pragma unroll
-    for (int t = 0; t < 2 * KS; ++t) acc[t] *= dn;
+    for (int t = 0; t < NT_; ++t) acc[t] *= dn;
 #pragma unroll
     for (int s = 0; s < 2; ++s) {
       const bf16x8_v bh =
@@ -422,11 +472,12 @@ qsa_retention_state(const bf16_t* __restrict__ x, long long xstride,
       const bf16x8_v bl =
           lds_frag_tr(vt[1], VP, s * 32, s * 32 + 16, wave * 16, lane);
 #pragma unroll
-      for (int t = 0; t < 2 * KS; ++t) {
+      for (int t = 0; t < NT_; ++t) {
+        const int d0 = (tile0 + t) * 16;
         const bf16x8_v ah =
-            lds_frag_tr(kt[0], KP, s * 32, s * 32 + 16, t * 16, lane);
+            lds_frag_tr(kt[0], KP, s * 32, s * 32 + 16, d0, lane);
         const bf16x8_v al =
-            lds_frag_tr(kt[1], KP, s * 32, s * 32 + 16, t * 16, lane);
+            lds_frag_tr(kt[1], KP, s * 32, s * 32 + 16, d0, lane);
         acc[t] = mfma_bf16(ah, bh, acc[t]);
         acc[t] = mfma_bf16(ah, bl, acc[t]);
         acc[t] = mfma_bf16(al, bh, acc[t]);
@@ -434,10 +485,10 @@ qsa_retention_state(const bf16_t* __restrict__ x, long long xstride,
     }
   }
 #pragma unroll
-  for (int t = 0; t < 2 * KS; ++t)
+  for (int t = 0; t < NT_; ++t)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int d = t * 16 + hi * 4 + r;
+      const int d = (tile0 + t) * 16 + hi * 4 + r;
       if (d < D && e < E) S[(long long)d * E + e] = acc[t][r];
     }
 }
@@ -448,29 +499,32 @@ extern "C" void qsa_retention_state_launch(
     const bf16_t* x, long long xstride, long long voff, const bf16_t* planes,
     long long rows, const float* log2_decay, float* state, const int* slots,
     const int* off, const int* start, const int* len, const int* chunk0,
-    bf16_t* prefix, long long n_chunks, int n_items, int H, int D, int DP,
-    int E, int EP, hipStream_t st) {
+    void* prefix, int n_items, int H, int D, int DP, int E, int EP,
+    hipStream_t st) {
   dim3 grid((unsigned)(n_items * H * ((EP + 63) / 64)));
-#define QSA_ST(K)                                                           \
+#define QSA_ST(K, DH)                                                       \
   case K:                                                                   \
-    hipLaunchKernelGGL((qsa_retention_state<K>), grid, dim3(256), 0, st, x, \
-                       xstride, voff, planes, rows, log2_decay, state,      \
-                       slots, off, start, len, chunk0, prefix, n_chunks, H, \
+    hipLaunchKernelGGL((qsa_retention_state<K, DH>), grid, dim3(256 * DH),  \
+                       0, st, x, xstride, voff, planes, rows, log2_decay, state,      \
+                       slots, off, start, len, chunk0, (u32x4_v*)prefix, H, \
                        D, E, EP);                                           \
     break;
-  switch (DP / 32) { QSA_ST(1) QSA_ST(2) QSA_ST(4) QSA_ST(8) }
+  switch (DP / 32) { QSA_ST(1, 1) QSA_ST(2, 2) QSA_ST(4, 2) QSA_ST(8, 2) }
 #undef QSA_ST
 }
 
 // ---------------------------------------------------------------------------
-// Step 3: outputs of one (chunk, head).  Wave w owns rows 16w..16w+15 and all
-// value columns, with O^T in accumulators (row = value, column = token):
+// Step 3: outputs of one (chunk, head) of 64 tokens, O^T in accumulators
+// (row = value, column = token):
 //   O^T  = decay^(i+1) * (S^T q_i)  +  V^T P^T,   P_ij = q_i.k_j decay^(i-j)
-// P^T leaves the first product in exactly the operand layout of the second
-// one (the order of the summed index is free), so nothing is shuffled.
+// Wave w of 8 owns the value tiles w, w+8, ... for all 64 tokens, so the state
+// before the chunk and V are read once per block.  For P, a wave computes 16
+// tokens against 32 keys; P^T leaves that product in
+// exactly the operand layout of the next one (the order of the summed index
+// is free) and passes through LDS, over the queries that are used up.
 // ---------------------------------------------------------------------------
 template <int KS, int ET>  // DP = 32*KS, up to 16*ET value columns
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(512)
 qsa_retention_out(const bf16_t* __restrict__ x, long long xstride,
                   long long voff, const bf16_t* __restrict__ planes,
                   long long rows, const float* __restrict__ log2_decay,
@@ -478,13 +532,16 @@ qsa_retention_out(const bf16_t* __restrict__ x, long long xstride,
                   const int* __restrict__ len,
                   const int* __restrict__ chunk_item,
                   const int* __restrict__ chunk_t0,
-                  const bf16_t* __restrict__ prefix, long long n_chunks,
+                  const u32x4_v* __restrict__ prefix,
                   bf16_t* __restrict__ out, int H, int E, int EP, float eps) {
   constexpr int DP = 32 * KS;
-  constexpr int KP = DP + 8;
+  constexpr int QP = DP + 8;
   constexpr int VP = 16 * ET + 16;
-  __shared__ __attribute__((aligned(16))) bf16_t kt[2][RC * KP];
+  constexpr int NV = ET <= 8 ? 1 : ET / 8;
+  constexpr int QSZ = RC * QP, PSZ = 2 * 2 * 4 * 64 * 8;
+  __shared__ __attribute__((aligned(16))) bf16_t qt[QSZ > PSZ ? QSZ : PSZ];
   __shared__ __attribute__((aligned(16))) bf16_t vt[RC * VP];
+  __shared__ float red[8][RC];
   const int h = blockIdx.x % H;
   const int ch = blockIdx.x / H;
   const int it = chunk_item[ch], t0 = chunk_t0[ch];
@@ -495,122 +552,170 @@ qsa_retention_out(const bf16_t* __restrict__ x, long long xstride,
   const int col = lane & 15, hi = lane >> 4;
   const float l2d = log2_decay[h];
   const long long plane = rows * H * DP;
+  const int NT = EP / 16;
 
-  // stage k planes and v
 #pragma unroll
-  for (int p = 0; p < 2; ++p)
-    for (int g = tid; g < RC * DP / 8; g += 256) {
-      const int row = g / (DP / 8), c = (g % (DP / 8)) * 8;
-      *reinterpret_cast<uint4*>(&kt[p][row * KP + c]) =
-          *reinterpret_cast<const uint4*>(
-              planes + (2 + p) * plane +
-              ((r0 + min(row, m - 1)) * H + h) * DP + c);
-    }
-  const int EG = (EP + 7) / 8;
-  for (int g = tid; g < RC * EG; g += 256) {
-    const int row = g / EG, c = (g % EG) * 8;
-    uint4 v = make_uint4(0, 0, 0, 0);
-    if (row < m && c < E)
-      v = *reinterpret_cast<const uint4*>(
-          x + (r0 + row) * xstride + voff + (long long)h * E + c);
-    *reinterpret_cast<uint4*>(&vt[row * VP + c]) = v;
+  for (int u = 0; u < (KS + 1) / 2; ++u) {
+    const int g = tid + u * 512;
+    if (KS == 1 && g >= RC * DP / 8) break;
+    const int row = g / (DP / 8), c = (g % (DP / 8)) * 8;
+    *reinterpret_cast<u32x4_v*>(&qt[row * QP + c]) =
+        *reinterpret_cast<const u32x4_v*>(
+            planes + ((r0 + min(row, m - 1)) * H + h) * DP + c);
   }
-  // this lane's token row i and its query operands
-  const int i = wave * 16 + col;
-  const long long qrow = r0 + min(i, m - 1);
-  bf16x8_v qh[KS], ql[KS];
 #pragma unroll
-  for (int s = 0; s < KS; ++s) {
-    const long long o = (qrow * H + h) * DP + s * 32 + hi * 8;
-    qh[s] = *reinterpret_cast<const bf16x8_v*>(planes + o);
-    ql[s] = *reinterpret_cast<const bf16x8_v*>(planes + plane + o);
+  for (int u = 0; u < ET / 4; ++u) {
+    const int g = tid + u * 512;
+    const int row = g / (2 * ET), c = (g % (2 * ET)) * 8;
+    const bool ok = row < m && c < E;               // E % 8 == 0
+    const u32x4_v v = *reinterpret_cast<const u32x4_v*>(
+        x + (r0 + min(row, m - 1)) * xstride + voff + (long long)h * E +
+        (c < E ? c : 0));
+    *reinterpret_cast<u32x4_v*>(&vt[row * VP + c]) =
+        ok ? v : (u32x4_v){0, 0, 0, 0};
   }
-  f32x4_v acc[ET];
+  f32x4_v acc[NV][4];
 #pragma unroll
-  for (int t = 0; t < ET; ++t) acc[t] = (f32x4_v){0.f, 0.f, 0.f, 0.f};
+  for (int u = 0; u < NV; ++u)
+#pragma unroll
+    for (int rt = 0; rt < 4; ++rt) acc[u][rt] = (f32x4_v){0.f, 0.f, 0.f, 0.f};
+  lds_barrier();
 
-  if (has_prefix) {                                   // uniform
-    const bf16_t* ph = prefix + ((long long)ch * H + h) * EP * DP;
-    const bf16_t* pl = ph + n_chunks * H * EP * DP;
+  if (has_prefix) {                                 // uniform
+    const u32x4_v* ph =
+        prefix + (((long long)ch * H + h) * 2) * NT * KS * 64 + lane;
+    const u32x4_v* pl = ph + (long long)NT * KS * 64;
 #pragma unroll
-    for (int t = 0; t < ET; ++t) {
-      if (t * 16 >= EP) break;                        // uniform
+    for (int s = 0; s < KS; ++s) {
+      bf16x8_v ah[NV], al[NV];
 #pragma unroll
-      for (int s = 0; s < KS; ++s) {
-        const int o = (t * 16 + col) * DP + s * 32 + hi * 8;
-        const bf16x8_v ah = *reinterpret_cast<const bf16x8_v*>(ph + o);
-        const bf16x8_v al = *reinterpret_cast<const bf16x8_v*>(pl + o);
-        acc[t] = mfma_bf16(ah, qh[s], acc[t]);
-        acc[t] = mfma_bf16(ah, ql[s], acc[t]);
-        acc[t] = mfma_bf16(al, qh[s], acc[t]);
+      for (int u = 0; u < NV; ++u) {
+        const int v = min(wave + 8 * u, NT - 1);    // spare tiles: not stored
+        ah[u] = __builtin_bit_cast(bf16x8_v, ph[(v * KS + s) * 64]);
+        al[u] = __builtin_bit_cast(bf16x8_v, pl[(v * KS + s) * 64]);
+      }
+#pragma unroll
+      for (int rt = 0; rt < 4; ++rt) {
+        const bf16_t* qr = &qt[(rt * 16 + col) * QP + s * 32 + hi * 4];
+        const bf16x8_v b = __builtin_shufflevector(
+            *reinterpret_cast<const bf16x4_v*>(qr),
+            *reinterpret_cast<const bf16x4_v*>(qr + 16), 0, 1, 2, 3, 4, 5, 6,
+            7);
+#pragma unroll
+        for (int u = 0; u < NV; ++u) {
+          acc[u][rt] = mfma_bf16(ah[u], b, acc[u][rt]);
+          acc[u][rt] = mfma_bf16(al[u], b, acc[u][rt]);
+        }
       }
     }
-    const float f = exp2f((float)(i + 1) * l2d);
 #pragma unroll
-    for (int t = 0; t < ET; ++t) acc[t] *= f;
+    for (int rt = 0; rt < 4; ++rt) {
+      const float f = exp2f((float)(rt * 16 + col + 1) * l2d);
+#pragma unroll
+      for (int u = 0; u < NV; ++u) acc[u][rt] *= f;
+    }
   }
-  __syncthreads();
 
-  // keys up to this wave's last row, 32 at a time
-  const int pairs = (wave >> 1) + 1;
-  for (int s2 = 0; s2 < pairs; ++s2) {
-    bf16x8_v pbh, pbl;
+  // P^T of token tile prt against key tiles 2*ps and 2*ps + 1, keys straight
+  // from the planes
+  const int prt = wave & 3, ps = wave >> 2;
+  const int i = prt * 16 + col;
+  u32x4_v pbh, pbl;
+  {
+    bf16x8_v q[KS];
+#pragma unroll
+    for (int s = 0; s < KS; ++s)
+      q[s] = *reinterpret_cast<const bf16x8_v*>(
+          &qt[i * QP + s * 32 + hi * 8]);
+    uint2 ph[2], pl[2];
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
-      const int pt = s2 * 2 + u;
+      const int pt = ps * 2 + u;
       f32x4_v sc = {0.f, 0.f, 0.f, 0.f};
+      if (pt <= prt) {                              // uniform over the wave
+        const bf16_t* kr = planes + plane +
+            ((r0 + min(pt * 16 + col, m - 1)) * H + h) * DP + hi * 8;
 #pragma unroll
-      for (int s = 0; s < KS; ++s) {
-        const int o = (pt * 16 + col) * KP + s * 32 + hi * 8;
-        const bf16x8_v ah = *reinterpret_cast<const bf16x8_v*>(&kt[0][o]);
-        const bf16x8_v al = *reinterpret_cast<const bf16x8_v*>(&kt[1][o]);
-        sc = mfma_bf16(ah, qh[s], sc);
-        sc = mfma_bf16(ah, ql[s], sc);
-        sc = mfma_bf16(al, qh[s], sc);
+        for (int s = 0; s < KS; ++s) {
+          const bf16x8_v ah = *reinterpret_cast<const bf16x8_v*>(kr + s * 32);
+          const bf16x8_v al =
+              *reinterpret_cast<const bf16x8_v*>(kr + plane + s * 32);
+          sc = mfma_bf16(ah, q[s], sc);
+          sc = mfma_bf16(al, q[s], sc);
+        }
       }
+      float w[4];
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int j = pt * 16 + hi * 4 + r;
-        const float f = (j <= i && j < m) ? exp2f((float)(i - j) * l2d) : 0.f;
-        bf16_t a, b;
-        split_bf16(j <= i && j < m ? sc[r] * f : 0.f, a, b);
-        pbh[u * 4 + r] = (short)a;
-        pbl[u * 4 + r] = (short)b;
+        const bool ok = j <= i && j < m;
+        w[r] = ok ? sc[r] * exp2f((float)(i - j) * l2d) : 0.f;
+      }
+      split4_bf16(w[0], w[1], w[2], w[3], ph[u], pl[u]);
+    }
+    pbh = (u32x4_v){ph[0].x, ph[0].y, ph[1].x, ph[1].y};
+    pbl = (u32x4_v){pl[0].x, pl[0].y, pl[1].x, pl[1].y};
+  }
+  lds_barrier();                                    // all queries are read
+  u32x4_v* pt = reinterpret_cast<u32x4_v*>(qt);     // [plane][s2][rt][lane]
+  pt[wave * 64 + lane] = pbh;
+  pt[(8 + wave) * 64 + lane] = pbl;
+  lds_barrier();
+#pragma unroll
+  for (int s2 = 0; s2 < 2; ++s2)
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      const int v = min(wave + 8 * u, NT - 1);
+      const bf16x8_v av = lds_frag_tr(vt, VP, s2 * 32, s2 * 32 + 16, v * 16,
+                                      lane);
+#pragma unroll
+      for (int rt = 2 * s2; rt < 4; ++rt) {
+        const bf16x8_v bh = __builtin_bit_cast(
+            bf16x8_v, pt[(s2 * 4 + rt) * 64 + lane]);
+        const bf16x8_v bl = __builtin_bit_cast(
+            bf16x8_v, pt[(8 + s2 * 4 + rt) * 64 + lane]);
+        acc[u][rt] = mfma_bf16(av, bh, acc[u][rt]);
+        acc[u][rt] = mfma_bf16(av, bl, acc[u][rt]);
       }
     }
-#pragma unroll
-    for (int t = 0; t < ET; ++t) {
-      if (t * 16 >= EP) break;
-      const bf16x8_v av =
-          lds_frag_tr(vt, VP, s2 * 32, s2 * 32 + 16, t * 16, lane);
-      acc[t] = mfma_bf16(av, pbh, acc[t]);
-      acc[t] = mfma_bf16(av, pbl, acc[t]);
-    }
-  }
 
   // per-token rms over the value columns, gate, store
-  float ss = 0.f;
 #pragma unroll
-  for (int t = 0; t < ET; ++t)
+  for (int rt = 0; rt < 4; ++rt) {
+    float ss = 0.f;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) ss = fmaf(acc[t][r], acc[t][r], ss);
-  ss += __shfl_xor(ss, 16, QSA_WAVE);
-  ss += __shfl_xor(ss, 32, QSA_WAVE);
-  const float inv = 1.f / sqrtf(ss / (float)E + eps);
-  if (i < m) {
-    const bf16_t* g = x + (r0 + i) * xstride + voff + (long long)H * E +
-                      (long long)h * E;
-    bf16_t* orow = out + ((r0 + i) * H + h) * E;
-#pragma unroll
-    for (int t = 0; t < ET; ++t) {
-      const int e0 = t * 16 + hi * 4;
-      if (e0 < E) {                                   // E % 8 == 0
-        float gv[4], o[4];
-        ldv<bf16_t, 4>(g + e0, gv);
+    for (int u = 0; u < NV; ++u)
+      if (wave + 8 * u < NT) {
 #pragma unroll
         for (int r = 0; r < 4; ++r)
-          o[r] = acc[t][r] * inv * (gv[r] / (1.f + __expf(-gv[r])));
-        stv<bf16_t, 4>(orow + e0, o);
+          ss = fmaf(acc[u][rt][r], acc[u][rt][r], ss);
+      }
+    ss += __shfl_xor(ss, 16, QSA_WAVE);
+    ss += __shfl_xor(ss, 32, QSA_WAVE);
+    if (hi == 0) red[wave][rt * 16 + col] = ss;
+  }
+  lds_barrier();
+#pragma unroll
+  for (int rt = 0; rt < 4; ++rt) {
+    const int t = rt * 16 + col;
+    const float ss = ((red[0][t] + red[1][t]) + (red[2][t] + red[3][t])) +
+                     ((red[4][t] + red[5][t]) + (red[6][t] + red[7][t]));
+    const float inv = 1.f / sqrtf(ss / (float)E + eps);
+    if (t < m) {
+      const bf16_t* g = x + (r0 + t) * xstride + voff + (long long)H * E +
+                        (long long)h * E;
+      bf16_t* orow = out + ((r0 + t) * H + h) * E;
+#pragma unroll
+      for (int u = 0; u < NV; ++u) {
+        const int e0 = (wave + 8 * u) * 16 + hi * 4;
+        if (e0 < E) {                               // E % 8 == 0
+          float gv[4], o[4];
+          ldv<bf16_t, 4>(g + e0, gv);
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+            o[r] = acc[u][rt][r] * inv * (gv[r] / (1.f + __expf(-gv[r])));
+          stv<bf16_t, 4>(orow + e0, o);
+        }
       }
     }
   }
@@ -620,17 +725,16 @@ extern "C" void qsa_retention_out_launch(
     const bf16_t* x, long long xstride, long long voff, const bf16_t* planes,
     long long rows, const float* log2_decay, const int* off,
     const int* start, const int* len, const int* chunk_item,
-    const int* chunk_t0, const bf16_t* prefix, long long n_chunks,
+    const int* chunk_t0, const void* prefix, long long n_chunks,
     bf16_t* out, int H, int DP, int E, int EP, float eps, hipStream_t st) {
   dim3 grid((unsigned)(n_chunks * H));
 #define QSA_RO(K, V)                                                        \
-  hipLaunchKernelGGL((qsa_retention_out<K, V>), grid, dim3(256), 0, st, x,  \
+  hipLaunchKernelGGL((qsa_retention_out<K, V>), grid, dim3(512), 0, st, x,  \
                      xstride, voff, planes, rows, log2_decay, off, start,   \
-                     len, chunk_item, chunk_t0, prefix, n_chunks, out, H,   \
-                     E, EP, eps)
+                     len, chunk_item, chunk_t0, (const u32x4_v*)prefix,     \
+                     out, H, E, EP, eps)
 #define QSA_RO_E(K)                                                         \
-  if (EP <= 32) QSA_RO(K, 2);                                               \
-  else if (EP <= 64) QSA_RO(K, 4);                                          \
+  if (EP <= 64) QSA_RO(K, 4);                                               \
   else if (EP <= 128) QSA_RO(K, 8);                                         \
   else if (EP <= 256) QSA_RO(K, 16);                                        \
   else QSA_RO(K, 32)
