@@ -1,8 +1,8 @@
 """Model registry: preset names and checkpoint folders -> decoder instances.
 
-BASELINE.json configs name two decoder families: Llama-3-8B (config 3, the
-flagship agent LLM) and Mixtral-8x7B MoE (config 5); Luzalorn is a
-config-driven decoder of retention and latent-attention layers.
+Three decoder families: Llama (Llama-3-8B is the flagship agent LLM, the
+Qwen2 geometry shares its class), Mixtral MoE, and Luzalorn, a config-driven
+decoder of retention and latent-attention layers.
 
 `build_model(name)` takes a preset name (random weights) or a folder with
 config.json + model.safetensors; a folder's class is chosen by the

@@ -139,8 +139,10 @@ class LatentAttention:
         self.sink = shard.rows(get("sink"))
         self.out = Linear(shard.cols(get("o")))
         self.longest = None
+        # sizes of the flash kernel, and a gate slice it can read in words
         if uk.is_cuda and dtype == torch.bfloat16 and \
-                self.R % 8 == 0 and D.window_attn_ok(H, self.D, self.E):
+                (self.Q + self.R) % 4 == 0 and self.R % 8 == 0 and \
+                D.window_attn_ok(H, self.D, self.E):
             self.longest = self.absorb_max
             self.ukv = Linear(torch.cat([uk, uv]))
 

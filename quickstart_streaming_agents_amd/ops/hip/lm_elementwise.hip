@@ -13,14 +13,14 @@
 // thread; wider rows re-read the residual this thread wrote itself.
 // ---------------------------------------------------------------------------
 template <typename T, int VEC, bool LAYER>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(1024)
 qsa_residual_norm(float* __restrict__ res, const T* __restrict__ y,
                   long long ystride, const T* __restrict__ table,
                   const long long* __restrict__ ids, const T* __restrict__ vec,
                   const T* __restrict__ w, const T* __restrict__ b,
                   T* __restrict__ out, int W, int vocab, float eps, int init) {
   constexpr int CACHED = 8;
-  __shared__ float scratch[8];
+  __shared__ float scratch[16];
   const long long row = blockIdx.x;
   float* rr = res + row * W;
   const T* yr = y ? y + row * ystride : nullptr;
@@ -131,7 +131,9 @@ static void residual_norm_go(float* res, const void* y, long long ystride,
                              void* out, long long rows, int W, int vocab,
                              float eps, int init, hipStream_t st) {
   int threads = ((W + VEC - 1) / VEC + 63) / 64 * 64;
-  threads = threads > 256 ? 256 : threads;
+  // few rows: wide blocks, one round of loads; many rows: narrow ones
+  const int most = rows <= 256 ? 1024 : 256;
+  threads = threads > most ? most : threads;
   hipLaunchKernelGGL((qsa_residual_norm<T, VEC, LAYER>), dim3((unsigned)rows),
                      dim3(threads), 0, st, res, (const T*)y, ystride,
                      (const T*)table, ids, (const T*)vec, (const T*)w,

@@ -49,6 +49,12 @@ CONFIGS = {
         ff(lat(5, 40, 72, 64, 96, 130, 0.2), 160),
         ff(ret(2, 48, 80, 32, [0.9, 0.9995], 1e5), 224),
         ff(ret(3, 32, 40, 32, [1.0, 0.99, 0.75]), 128)]),
+    # sizes that fit one kernel's matrix-core form and not its neighbour's
+    "uneven": dict(vocab=130, width=72, norm={"eps": 1e-5},
+                   loop={"start": 1, "stop": 2, "times": 2}, layers=[
+        ff(lat(2, 32, 32, 50, 64, 90, 0.3), 50),
+        ff(ret(3, 10, 16, 6, [0.95, 0.9, 0.999]), 44),
+        ff(lat(3, 12, 32, 32, 520, 33, 0.4), 36)]),
     # one head each, the loop runs once, a window of one token, up to the end
     "ones": dict(vocab=96, width=64, norm={"eps": 1e-5},
                  loop={"start": 1, "stop": 3, "times": 1}, layers=[

@@ -26,6 +26,34 @@ def stats():
     return out
 
 
+@pytest.fixture(scope="module")
+def lm_stats():
+    import isa_check
+    so = isa_check.find_so("qsa_lm_hip")
+    if so is None or not os.path.exists(isa_check.BUNDLER):
+        pytest.skip("built extension or ROCm LLVM tools unavailable")
+    import tempfile
+    with tempfile.TemporaryDirectory() as wd:
+        out = isa_check.kernel_stats(isa_check.extract_hsacos(so, wd))
+    if not out:
+        pytest.skip("no gfx950 code objects extracted")
+    return out
+
+
+def test_mixer_kernels(lm_stats):
+    """Matrix kernels issue MFMA, nothing spills vector registers or uses
+    scratch, and no packed f32 arithmetic was formed."""
+    for frag in ("retention_state", "retention_out", "latent_rows_mfma",
+                 "window_attn_prefill", "head_matmul_mfma", "skinny_gemm"):
+        for name, st in _named(lm_stats, frag).items():
+            assert st["mfma"] >= 4, f"{name}: only {st['mfma']} v_mfma"
+    for name, st in lm_stats.items():
+        if name.startswith("_Z"):
+            assert st.get("vgpr_spill_count", 0) == 0, name
+            assert st.get("private_segment_fixed_size", 0) == 0, name
+            assert st.get("packed_f32", 0) == 0, name
+
+
 def _named(stats, frag):
     hits = {k: v for k, v in stats.items() if frag in k}
     assert hits, f"no kernel matching {frag!r}"
@@ -49,8 +77,8 @@ def test_no_spills_or_scratch_on_hot_kernels(stats):
                 f"{name}: scratch allocated"
 
 
-def test_round2_kernels_present_and_clean(stats):
-    """Round-2 kernels: fp8 GEMMs issue MFMA + the fp8 dequant path
+def test_fp8_and_join_kernels_present_and_clean(stats):
+    """The fp8 GEMMs issue MFMA + the fp8 dequant path
     (v_cvt_pk_f32_fp8); the hash-join kernels exist; none spill."""
     for frag in ("skinny_gemm_fp8", "gemm_fp8_batch"):
         hits = _named(stats, frag)

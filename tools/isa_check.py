@@ -22,10 +22,10 @@ TARGET = "hipv4-amdgcn-amd-amdhsa--gfx950"
 MAGIC = b"__CLANG_OFFLOAD_BUNDLE__"
 
 
-def find_so() -> str | None:
+def find_so(module: str = "qsa_hip") -> str | None:
     root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
     hits = glob.glob(os.path.join(
-        root, "quickstart_streaming_agents_amd", "qsa_hip*.so"))
+        root, "quickstart_streaming_agents_amd", module + ".*so"))
     return hits[0] if hits else None
 
 
@@ -76,6 +76,9 @@ def kernel_stats(hsacos: list[str]) -> dict[str, dict]:
                 stats[cur]["total"] += 1
                 if "v_mfma" in line:
                     stats[cur]["mfma"] += 1
+                elif re.search(r"v_pk_(add|mul|fma)_f32", line):
+                    stats[cur]["packed_f32"] = \
+                        stats[cur].get("packed_f32", 0) + 1
         notes = subprocess.run(
             [os.path.join(LLVM, "llvm-readelf"), "--notes", h],
             capture_output=True, text=True).stdout
@@ -92,12 +95,14 @@ def kernel_stats(hsacos: list[str]) -> dict[str, dict]:
 
 
 def main() -> int:
-    so = find_so()
-    if so is None:
+    found = [so for so in map(find_so, ("qsa_hip", "qsa_lm_hip")) if so]
+    if not found:
         print("no built extension found")
         return 1
-    with tempfile.TemporaryDirectory() as wd:
-        stats = kernel_stats(extract_hsacos(so, wd))
+    stats = {}
+    for so in found:
+        with tempfile.TemporaryDirectory() as wd:
+            stats.update(kernel_stats(extract_hsacos(so, wd)))
     for name, st in sorted(stats.items()):
         if st["total"] > 60:
             print(f"{name[:64]:64s} instr={st['total']:5d} "
