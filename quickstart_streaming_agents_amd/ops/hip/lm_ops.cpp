@@ -297,7 +297,7 @@ void retention_chunked(Tensor x, Tensor cos_t, Tensor sin_t,
   TORCH_CHECK(out.size(0) == T && out.size(1) == (long long)r.H * r.E, "out");
   if (n == 0 || nc == 0) return;
   const int DP = pad_dim(r.D), EP = (r.E + 15) / 16 * 16;
-  auto planes = torch::empty({3, T, r.H, DP}, x.options());
+  auto planes = torch::empty({4, T, r.H, DP}, x.options());
   auto prefix = torch::empty({nc, r.H, 2, EP, DP}, x.options());
   hipStream_t st = cur_stream();
   const long long voff = 2LL * r.H * r.D;

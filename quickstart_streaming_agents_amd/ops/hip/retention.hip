@@ -15,16 +15,16 @@
 //   qsa_retention_seq      token loop per (portion, head), any size and
 //                          storage type; the f32 path.
 //   chunked prefill (bf16 storage, matrix cores), chunks of 64 tokens:
-//     qsa_retention_rotate   rotated q (bf16) and k (bf16 hi/lo), padded
+//     qsa_retention_rotate   rotated q, k as bf16 hi/lo planes, zero-padded
 //     qsa_retention_state    walks the chunks of a portion, state tile in
 //                            accumulators; leaves the state before each
 //                            chunk as hi/lo matrix-core operands
 //     qsa_retention_out      per (chunk, head): inter-chunk read-out,
 //                            intra-chunk masked product, norm, gate
-// Everything that enters the recurrence is a bf16 hi/lo pair on the matrix
-// cores (k, the decayed v, the state, the intra-chunk weights), so the chunked
-// recurrence agrees with the token loop to ~2^-16; q, which only reads the
-// state out, is rounded once like any activation, and v is bf16 already.
+// Every rounded operand is a bf16 hi/lo pair on the matrix cores (q, k, the
+// decayed v, the state, the intra-chunk weights), so the chunked result agrees
+// with the token loop to ~2^-16; v is bf16 already.  One-sided rounding would
+// show: the norm over a head blows it up where S^T q is small.
 #include "lm_common.h"
 
 #define RC 64  // tokens per chunk
@@ -250,7 +250,7 @@ extern "C" void qsa_retention_seq_launch(
 }
 
 // ---------------------------------------------------------------------------
-// Chunked prefill, step 1: planes[p][row][h][DP], p = q, k.hi, k.lo
+// Chunked prefill, step 1: planes[p][row][h][DP], p = q.hi, q.lo, k.hi, k.lo
 // ---------------------------------------------------------------------------
 // One thread per 8 dims of a head of a row, q and k.  FAST: whole groups on
 // either side of the rotation pairs (rot % 16 == 0, D % 8 == 0, 16 B rows).
@@ -310,13 +310,15 @@ qsa_retention_rotate(const bf16_t* __restrict__ x, long long xstride,
     for (int j = 0; j < 8; ++j) kv[j] *= kscale;
     uint2 a0, b0, a1, b1;
     bf16_t* o = planes + (row * H + h) * DP + d0;
-    *reinterpret_cast<uint4*>(o) =
-        make_uint4(cvt_bf16x2(qv[0], qv[1]), cvt_bf16x2(qv[2], qv[3]),
-                   cvt_bf16x2(qv[4], qv[5]), cvt_bf16x2(qv[6], qv[7]));
+    split4_bf16(qv[0], qv[1], qv[2], qv[3], a0, b0);
+    split4_bf16(qv[4], qv[5], qv[6], qv[7], a1, b1);
+    *reinterpret_cast<uint4*>(o) = make_uint4(a0.x, a0.y, a1.x, a1.y);
+    *reinterpret_cast<uint4*>(o + plane) = make_uint4(b0.x, b0.y, b1.x, b1.y);
     split4_bf16(kv[0], kv[1], kv[2], kv[3], a0, b0);
     split4_bf16(kv[4], kv[5], kv[6], kv[7], a1, b1);
-    *reinterpret_cast<uint4*>(o + plane) = make_uint4(a0.x, a0.y, a1.x, a1.y);
     *reinterpret_cast<uint4*>(o + 2 * plane) =
+        make_uint4(a0.x, a0.y, a1.x, a1.y);
+    *reinterpret_cast<uint4*>(o + 3 * plane) =
         make_uint4(b0.x, b0.y, b1.x, b1.y);
   }
 }
@@ -381,7 +383,7 @@ qsa_retention_state(const bf16_t* __restrict__ x, long long xstride,
   const int e = v0 + wave * 16 + col;          // this lane's value column
   float* S = state + ((long long)slot * H + h) * D * E;
   const long long plane = rows * H * DP;
-  const bf16_t* kpl = planes + plane;
+  const bf16_t* kpl = planes + 2 * plane;
 
   f32x4_v acc[NT_];
 #pragma unroll
@@ -538,7 +540,7 @@ qsa_retention_out(const bf16_t* __restrict__ x, long long xstride,
   constexpr int QP = DP + 8;
   constexpr int VP = 16 * ET + 16;
   constexpr int NV = ET <= 8 ? 1 : ET / 8;
-  constexpr int QSZ = RC * QP, PSZ = 2 * 2 * 4 * 64 * 8;
+  constexpr int QSZ = 2 * RC * QP, PSZ = 2 * 2 * 4 * 64 * 8;
   __shared__ __attribute__((aligned(16))) bf16_t qt[QSZ > PSZ ? QSZ : PSZ];
   __shared__ __attribute__((aligned(16))) bf16_t vt[RC * VP];
   __shared__ float red[8][RC];
@@ -555,13 +557,13 @@ qsa_retention_out(const bf16_t* __restrict__ x, long long xstride,
   const int NT = EP / 16;
 
 #pragma unroll
-  for (int u = 0; u < (KS + 1) / 2; ++u) {
-    const int g = tid + u * 512;
-    if (KS == 1 && g >= RC * DP / 8) break;
-    const int row = g / (DP / 8), c = (g % (DP / 8)) * 8;
-    *reinterpret_cast<u32x4_v*>(&qt[row * QP + c]) =
+  for (int u = 0; u < KS; ++u) {
+    const int g = tid + u * 512;                    // plane, row, group
+    const int p = g / (RC * DP / 8);
+    const int row = g / (DP / 8) % RC, c = (g % (DP / 8)) * 8;
+    *reinterpret_cast<u32x4_v*>(&qt[(p * RC + row) * QP + c]) =
         *reinterpret_cast<const u32x4_v*>(
-            planes + ((r0 + min(row, m - 1)) * H + h) * DP + c);
+            planes + p * plane + ((r0 + min(row, m - 1)) * H + h) * DP + c);
   }
 #pragma unroll
   for (int u = 0; u < ET / 4; ++u) {
@@ -597,14 +599,19 @@ qsa_retention_out(const bf16_t* __restrict__ x, long long xstride,
 #pragma unroll
       for (int rt = 0; rt < 4; ++rt) {
         const bf16_t* qr = &qt[(rt * 16 + col) * QP + s * 32 + hi * 4];
-        const bf16x8_v b = __builtin_shufflevector(
+        const bf16x8_v bh = __builtin_shufflevector(
             *reinterpret_cast<const bf16x4_v*>(qr),
             *reinterpret_cast<const bf16x4_v*>(qr + 16), 0, 1, 2, 3, 4, 5, 6,
             7);
+        const bf16x8_v bl = __builtin_shufflevector(
+            *reinterpret_cast<const bf16x4_v*>(qr + RC * QP),
+            *reinterpret_cast<const bf16x4_v*>(qr + RC * QP + 16), 0, 1, 2, 3,
+            4, 5, 6, 7);
 #pragma unroll
         for (int u = 0; u < NV; ++u) {
-          acc[u][rt] = mfma_bf16(ah[u], b, acc[u][rt]);
-          acc[u][rt] = mfma_bf16(al[u], b, acc[u][rt]);
+          acc[u][rt] = mfma_bf16(ah[u], bh, acc[u][rt]);
+          acc[u][rt] = mfma_bf16(ah[u], bl, acc[u][rt]);
+          acc[u][rt] = mfma_bf16(al[u], bh, acc[u][rt]);
         }
       }
     }
@@ -622,26 +629,29 @@ qsa_retention_out(const bf16_t* __restrict__ x, long long xstride,
   const int i = prt * 16 + col;
   u32x4_v pbh, pbl;
   {
-    bf16x8_v q[KS];
+    bf16x8_v qh[KS], ql[KS];
 #pragma unroll
-    for (int s = 0; s < KS; ++s)
-      q[s] = *reinterpret_cast<const bf16x8_v*>(
-          &qt[i * QP + s * 32 + hi * 8]);
+    for (int s = 0; s < KS; ++s) {
+      const bf16_t* qr = &qt[i * QP + s * 32 + hi * 8];
+      qh[s] = *reinterpret_cast<const bf16x8_v*>(qr);
+      ql[s] = *reinterpret_cast<const bf16x8_v*>(qr + RC * QP);
+    }
     uint2 ph[2], pl[2];
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
       const int pt = ps * 2 + u;
       f32x4_v sc = {0.f, 0.f, 0.f, 0.f};
       if (pt <= prt) {                              // uniform over the wave
-        const bf16_t* kr = planes + plane +
+        const bf16_t* kr = planes + 2 * plane +
             ((r0 + min(pt * 16 + col, m - 1)) * H + h) * DP + hi * 8;
 #pragma unroll
         for (int s = 0; s < KS; ++s) {
           const bf16x8_v ah = *reinterpret_cast<const bf16x8_v*>(kr + s * 32);
           const bf16x8_v al =
               *reinterpret_cast<const bf16x8_v*>(kr + plane + s * 32);
-          sc = mfma_bf16(ah, q[s], sc);
-          sc = mfma_bf16(al, q[s], sc);
+          sc = mfma_bf16(ah, qh[s], sc);
+          sc = mfma_bf16(ah, ql[s], sc);
+          sc = mfma_bf16(al, qh[s], sc);
         }
       }
       float w[4];
