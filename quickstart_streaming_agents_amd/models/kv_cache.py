@@ -3,7 +3,8 @@
 `PageAllocator` hands out 64-position pages; one page-id space spans all
 layers, so a sequence has ONE page list used by every layer.
 
-`PagedKVCache` (Llama, Mixtral) stores keys and values in the layouts of ops/hip/paged_attn.hip:
+`PagedKVCache` (Llama, Mixtral) stores keys and values in the layouts of
+ops/hip/paged_attn.hip:
   K: [pages, KVH, D/8, 64, 8]  (d-major x8 -> coalesced MFMA A-frag reads)
   V: [pages, KVH, D, 64]       (transposed, pos minor -> coalesced MFMA
                                 B-frag reads in the PV pass)
