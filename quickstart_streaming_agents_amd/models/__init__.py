@@ -1,8 +1,9 @@
 """Model registry: preset names and checkpoint folders -> decoder instances.
 
-Three decoder families: Llama (Llama-3-8B is the flagship agent LLM, the
-Qwen2 geometry shares its class), Mixtral MoE, and Luzalorn, a config-driven
-decoder of retention and latent-attention layers.
+Decoder families: Llama (Llama-3-8B is the flagship agent LLM, the Qwen2
+geometry shares its class), Mixtral MoE, and the config-driven mixer decoders:
+Luzalorn (retention and latent-attention layers) and Lunulix (attention and a
+state-space layer side by side).
 
 `build_model(name)` takes a preset name (random weights) or a folder with
 config.json + model.safetensors; a folder's class is chosen by the
@@ -20,8 +21,14 @@ def _luzalorn():
     return LuzalornModel
 
 
-# config.json 'architecture' -> loader of the model class
-ARCHITECTURES = {"Luzalorn": _luzalorn}
+def _lunulix():
+    from .lunulix import LunulixModel
+    return LunulixModel
+
+
+# config.json 'architecture' -> loader of the model class; a preset of the
+# family is named after it ("luzalorn-8b", "tiny-lunulix")
+ARCHITECTURES = {"Luzalorn": _luzalorn, "Lunulix": _lunulix}
 
 
 def load_model(folder: str, device: str = "cuda", dtype=None, **kw):
@@ -49,10 +56,11 @@ def build_model(name: str, device: str = "cuda", dtype=None, seed: int = 0,
     tp = dict(tp_rank=tp_rank, tp_size=tp_size, tp_group=tp_group)
     if os.path.isfile(os.path.join(name, "config.json")):
         return load_model(name, device=device, dtype=dtype, **tp)
-    if name.startswith("luzalorn") or name == "tiny-luzalorn":
-        from .luzalorn import LuzalornConfig, LuzalornModel
-        return LuzalornModel(LuzalornConfig.preset(name), device=device,
-                             dtype=dtype, seed=seed, **tp)
+    for arch, cls in ARCHITECTURES.items():
+        if arch.lower() in name.split("-"):
+            model = cls()
+            return model(model.Config.preset(name), device=device,
+                         dtype=dtype, seed=seed, **tp)
     if name.startswith("mixtral") or name == "tiny-moe":
         from .mixtral import MixtralConfig, MixtralModel
         return MixtralModel(MixtralConfig.preset(name), device=device,

@@ -12,7 +12,12 @@ ops/hip/paged_attn.hip:
 `HybridCache` serves decoders that mix attention with recurrent layers:
   latents: [pages, 64, rank] per attention run (ops/hip/latent_attn.hip)
   states:  [slots, heads, dim, vdim] f32 per recurrent run
-           (ops/hip/retention.hip), one slot per live sequence
+           (ops/hip/retention.hip, ssd.hip), one slot per live sequence
+A recurrent run may also hold, at the same index,
+  keys:    [pages, kv heads, 64, dim] and values [pages, kv heads, 64, vdim]
+           (ops/hip/gqa_attn.hip), for a mixer that attends beside its state
+  tails:   [slots, taps - 1, channels] per short convolution, its last inputs
+           (ops/hip/short_conv.hip); they share the sequence's slot
 A "run" is one execution of a layer: a layer that a loop repeats has a cache
 or state of its own for every pass.
 """
@@ -126,7 +131,7 @@ class PagedKVCache(PageAllocator):
 
 
 class HybridCache(PageAllocator):
-    """Pages of latents plus state slots.
+    """Pages of latents or keys and values, plus state slots.
 
     Unlike pages, a recurrent state cannot be rolled back to an arbitrary
     earlier position.  A conversation therefore takes a snapshot() when its
@@ -145,13 +150,25 @@ class HybridCache(PageAllocator):
     def __init__(self, n_pages: int, n_slots: int,
                  latent_ranks: list[int],
                  state_shapes: list[tuple[int, int, int]],
-                 device: str = "cuda", dtype=torch.bfloat16):
+                 device: str = "cuda", dtype=torch.bfloat16,
+                 kv_shapes: list[tuple[int, int, int] | None] = (),
+                 tail_shapes: list[tuple[tuple[int, int], ...]] = ()):
+        """kv_shapes (kv heads, dim, vdim) or None, and tail_shapes, one
+        (taps - 1, channels) per convolution, go with state_shapes."""
         super().__init__(n_pages, device)
         self.n_slots = n_slots
         self.latents = [torch.zeros(n_pages, self.PAGE, r, dtype=dtype,
                                     device=device) for r in latent_ranks]
         self.states = [torch.zeros(n_slots, *s, dtype=torch.float32,
                                    device=device) for s in state_shapes]
+        paged = [s and [torch.zeros(n_pages, s[0], self.PAGE, d, dtype=dtype,
+                                    device=device) for d in s[1:]]
+                 for s in kv_shapes]
+        self.keys = [p and p[0] for p in paged]
+        self.values = [p and p[1] for p in paged]
+        self.tails = [tuple(torch.zeros(n_slots, *t, dtype=dtype,
+                                        device=device) for t in ts)
+                      for ts in tail_shapes]
         self._free_slots = list(range(n_slots - 1, -1, -1))
         self._slot: dict[int, int] = {}
         self._snap: dict[int, tuple[int, int]] = {}    # seq -> (slot, len)
@@ -212,7 +229,7 @@ class HybridCache(PageAllocator):
         if not self._free_slots and not self._parked:
             return                         # no room: the next turn re-reads
         dst, src = self._take_slot(), self._slot[seq_id]
-        for s in self.states:
+        for s in (*self.states, *(t for ts in self.tails for t in ts)):
             s[dst].copy_(s[src])
         self._snap[seq_id] = (dst, self._seq_len[seq_id])
 

@@ -3,6 +3,8 @@ tables, feed-forwards and the device-side description of a step."""
 
 from __future__ import annotations
 
+import math
+
 import numpy as np
 import torch
 import torch.nn.functional as F
@@ -34,13 +36,35 @@ class Linear:
         return F.linear(x, self.w)
 
 
-class RopeTable:
-    """cos/sin of p * base^(-2i/dims), [positions, dims/2] f32, evaluated in
-    f64.  Grows on demand; earlier tables stay alive because a captured
-    graph may still read them."""
+def rope_frequencies(dims: int, base: float,
+                     scaling: dict | None = None) -> torch.Tensor:
+    """Angle per position of each rotated pair, base^(-2i/dims) in f64.
+    `scaling` (factor, low, high, original) stretches a model's context as
+    Llama 3.1 does: wavelengths beyond original/low are slowed down by factor,
+    those under original/high kept, and the ones between blended."""
+    f = base ** (-2.0 * torch.arange(dims // 2, dtype=torch.float64)
+                 / max(dims, 1))
+    if not scaling:
+        return f
+    n, low, high = (float(scaling[k]) for k in ("original", "low", "high"))
+    slow = f / float(scaling["factor"])
+    wave = 2.0 * math.pi / f
+    s = (n / wave - low) / (high - low) if high != low \
+        else torch.zeros_like(f)
+    out = (1.0 - s) * slow + s * f
+    out = torch.where(wave > n / low, slow, out)
+    return torch.where(wave < n / high, f, out)
 
-    def __init__(self, dims: int, base: float, device: str):
+
+class RopeTable:
+    """cos/sin of p * frequency, [positions, dims/2] f32, evaluated in f64.
+    Grows on demand; earlier tables stay alive because a captured graph may
+    still read them."""
+
+    def __init__(self, dims: int, base: float, device: str,
+                 scaling: dict | None = None):
         self.dims, self.base, self.device = dims, base, device
+        self.freq = rope_frequencies(dims, base, scaling)
         self._kept: list[torch.Tensor] = []
         self.cos = self.sin = torch.zeros(0, dims // 2, device=device)
 
@@ -48,27 +72,39 @@ class RopeTable:
         if n <= self.cos.shape[0]:
             return
         n = max(256, 1 << (n - 1).bit_length())
-        half = self.dims // 2
-        inv = self.base ** (-2.0 * torch.arange(half, dtype=torch.float64)
-                            / max(self.dims, 1))
-        ang = torch.outer(torch.arange(n, dtype=torch.float64), inv)
+        ang = torch.outer(torch.arange(n, dtype=torch.float64), self.freq)
         self._kept += [self.cos, self.sin]
         self.cos = ang.cos().float().to(self.device)
         self.sin = ang.sin().float().to(self.device)
 
 
 class DenseGLU:
-    """W_down(silu(W_gate h) * (W_up h)); gate and up share one GEMM."""
+    """W_down(act(W_gate h) * (W_up h)); gate and up share one GEMM."""
 
     def __init__(self, gate: torch.Tensor, up: torch.Tensor,
-                 down: torch.Tensor):
-        self.ff = gate.shape[0]
+                 down: torch.Tensor, act: str = "silu"):
+        self.ff, self.act = gate.shape[0], act
         self.gate_up = Linear(torch.cat([gate, up]).contiguous())
         self.down = Linear(down)
 
     def __call__(self, h: torch.Tensor) -> torch.Tensor:
         gu = self.gate_up(h)
-        return self.down(D.glu(gu[:, :self.ff], gu[:, self.ff:]))
+        return self.down(D.glu(gu[:, :self.ff], gu[:, self.ff:], self.act))
+
+
+class TokenSide:
+    """Per-layer input of the token itself: W_proj(act(W_gate x) * e), e the
+    layer's columns of the token's row in a table that all layers share."""
+
+    def __init__(self, gate: torch.Tensor, proj: torch.Tensor,
+                 table: torch.Tensor, layer: int, act: str = "gelu"):
+        self.table, self.act = table, act
+        self.col0 = layer * gate.shape[0]
+        self.gate, self.proj = Linear(gate), Linear(proj)
+
+    def __call__(self, x: torch.Tensor, ids: torch.Tensor) -> torch.Tensor:
+        return self.proj(D.glu_table(self.gate(x), self.table, ids,
+                                     self.col0, self.act))
 
 
 def ints_to_device(device, *arrays: np.ndarray) -> list[torch.Tensor]:
@@ -97,6 +133,15 @@ class AttnPortions:
         self.ctx_slots = ctx_slots
 
 
+class PagedPortions:
+    """Portions whose queries go over the pages block by block."""
+
+    def __init__(self, qb_item, qb_t0, off, start, length, table):
+        self.qb_item, self.qb_t0 = qb_item, qb_t0
+        self.off, self.start, self.length = off, start, length
+        self.table = table
+
+
 class StepPlan:
     """Device-side description of one engine step.
 
@@ -104,8 +149,11 @@ class StepPlan:
     by length, so every kernel family works on one contiguous row range:
     rows [0, n_one) advance a sequence by one token, the rest are portions
     of at least two tokens.  `order` maps the plan's entries back to the
-    caller's.
+    caller's.  `conv` describes all rows to the short convolutions: portions
+    in chunks of CONV_ROWS rows, or single tokens (ops.dispatch.conv_qkv).
     """
+
+    CONV_ROWS = 16
 
     def __init__(self):
         self._rows: dict = {}
@@ -121,6 +169,7 @@ class StepPlan:
         p.one_lens = seq_lens
         p.one_slots = state_slots
         p.cache_slots = D.decode_slots(block_table, seq_lens)
+        p.conv = (None, None, None, seq_lens, None, state_slots)
         p.items = None
         return p
 
@@ -156,14 +205,25 @@ class StepPlan:
         ch_item = np.repeat(np.arange(len(nch)), nch)
         ch_t0 = (np.arange(int(nch.sum())) - chunk0[ch_item]) * 64 \
             if len(nch) else np.zeros(0)
+        cv_item, cv_t0 = cls._cut(lens, cls.CONV_ROWS)
         (bt, p.cache_slots, p.one_slots, p.one_lens, p.p_slots, p.p_off,
          p.p_start, p.p_len, p.p_pos, p.chunk0, p.chunk_item,
-         p.chunk_t0) = ints_to_device(
+         p.chunk_t0, *conv) = ints_to_device(
             dev, table.reshape(-1), slot_ids, state[:n1], starts[:n1] + 1,
             state[n1:], p.offs[n1:-1] - n1, starts[n1:], lens[n1:], pos[n1:],
-            chunk0, ch_item, ch_t0)
+            chunk0, ch_item, ch_t0, cv_item, cv_t0, p.offs[:-1], starts, lens,
+            state)
+        p.conv = tuple(conv)
         p.block_table = bt.view(len(items), cap)
         return p
+
+    @staticmethod
+    def _cut(lens, size: int):
+        """(entry, first token) of pieces of at most `size` tokens."""
+        n = -(-lens // size)
+        item = np.repeat(np.arange(len(lens)), n)
+        return item, (np.arange(int(n.sum()))
+                      - (np.cumsum(n) - n)[item]) * size
 
     # ---- attention routes ------------------------------------------------
     def attn_rows(self, longest: int | None) -> AttnRows:
@@ -208,4 +268,26 @@ class StepPlan:
             self._portions[key] = AttnPortions(*ints_to_device(
                 self.device, qb_item, qb_t0, self.offs[k:-1] - self.offs[k],
                 starts, lens, ctx_off, first, np.concatenate(ctx)))
+        return self._portions[key]
+
+    def paged_portions(self, longest: int | None,
+                       rows: int) -> PagedPortions | None:
+        """Entries of more than `longest` tokens in blocks of `rows` query
+        rows, the ones with most keys first; row offsets count from the first
+        of their rows."""
+        if self.items is None or longest is None:
+            return None
+        key = ("paged", longest, rows)
+        if key not in self._portions:
+            k = int((self.lens <= longest).sum())
+            lens, starts = self.lens[k:], self.starts[k:]
+            if not len(lens):
+                self._portions[key] = None
+                return None
+            item, t0 = self._cut(lens, rows)
+            heavy = np.argsort(-(starts[item] + t0), kind="stable")
+            self._portions[key] = PagedPortions(*ints_to_device(
+                self.device, item[heavy], t0[heavy],
+                self.offs[k:-1] - self.offs[k], starts, lens),
+                self.block_table[k:])
         return self._portions[key]

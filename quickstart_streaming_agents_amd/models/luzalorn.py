@@ -18,16 +18,15 @@ sizes and 'mlp'); the mixers are models/mixers.py.
 
 from __future__ import annotations
 
-import os
 from dataclasses import dataclass
 
 import torch
 
 from ..ops import dispatch as D
+from .decoder import LayerRun, MixerDecoder, check_layers, number_runs
 from .kv_cache import HybridCache
-from .layers import DenseGLU, Linear, RopeTable, StepPlan
-from .mixers import MIXERS, Shard
-from .weights import SafetensorsFile
+from .layers import DenseGLU, Linear, StepPlan
+from .mixers import MIXERS
 
 
 @dataclass
@@ -42,12 +41,7 @@ class LuzalornConfig:
 
     def __post_init__(self):
         n = len(self.layers)
-        for i, L in enumerate(self.layers):
-            if L["type"] not in MIXERS:
-                raise ValueError(f"layer {i}: unknown mixer {L['type']!r}")
-            if L.get("mlp") and L["mlp"].get("kind", "dense") != "dense":
-                raise ValueError(f"layer {i}: unknown feed-forward "
-                                 f"{L['mlp']['kind']!r}")
+        check_layers(self.layers)
         if self.loop:
             a, b = self.loop["start"], self.loop["stop"]
             if not (0 <= a < b <= n and self.loop["times"] >= 1):
@@ -156,16 +150,7 @@ class _Layer:
     ff: DenseGLU | None = None
 
 
-@dataclass
-class _Run:
-    """One execution of a layer."""
-    layer: int
-    cache: int                   # index among the runs of its kind
-    step: int | None = None      # first layer of pass t: add loop.step[t]
-    re_embed: bool = False       # ... and the embedding output
-
-
-def layer_runs(c: LuzalornConfig) -> list[_Run]:
+def layer_runs(c: LuzalornConfig) -> list[LayerRun]:
     n = len(c.layers)
     seq: list[tuple[int, int | None]] = []
     if c.loop:
@@ -176,40 +161,17 @@ def layer_runs(c: LuzalornConfig) -> list[_Run]:
         seq += [(i, None) for i in range(b, n)]
     else:
         seq = [(i, None) for i in range(n)]
-    count: dict[str, int] = {}
-    runs = []
-    for i, t in seq:
-        kind = c.layers[i]["type"]
-        k = count.get(kind, 0)
-        count[kind] = k + 1
-        runs.append(_Run(i, k, step=t, re_embed=t is not None and t > 0))
-    return runs
+    return number_runs(c.layers, seq)
 
 
-class LuzalornModel:
-    def __init__(self, cfg: LuzalornConfig, device: str = "cuda",
-                 dtype=torch.bfloat16, seed: int = 0, weights=None,
-                 tp_rank: int = 0, tp_size: int = 1, tp_group=None):
-        """weights: name -> tensor mapping (a dict or SafetensorsFile);
-        without it, random weights from `seed`."""
-        self.cfg, self.device, self.dtype = cfg, device, dtype
-        self.tp_rank, self.tp_size, self.tp_group = tp_rank, tp_size, tp_group
-        self.runs = layer_runs(cfg)
-        self.shard = shard = Shard(tp_rank, tp_size)
-        self._ropes: dict[tuple[int, float], RopeTable] = {}
-        shapes = tensor_shapes(cfg)
-        if weights is None:
-            weights = dict(random_weights(cfg, device, dtype, seed))
+class LuzalornModel(MixerDecoder):
+    Config = LuzalornConfig
+    shapes = staticmethod(tensor_shapes)
+    random = staticmethod(random_weights)
+    layer_runs = staticmethod(layer_runs)
 
-        def get(name: str) -> torch.Tensor:
-            t = weights.get(name)
-            if t is None:
-                raise KeyError(f"checkpoint has no tensor {name!r}")
-            if tuple(t.shape) != shapes[name]:
-                raise ValueError(f"{name}: shape {tuple(t.shape)}, the "
-                                 f"configuration asks for {shapes[name]}")
-            return t.to(device=device, dtype=dtype).contiguous()
-
+    def build(self, get) -> None:
+        cfg, shard = self.cfg, self.shard
         self.embed = get("embed")
         self.head = Linear(self.embed)
         self.loop_step = get("loop.step") if cfg.loop else None
@@ -221,59 +183,18 @@ class LuzalornModel:
                 (get(p + "norm1"), get(p + "norm1.b")),
                 MIXERS[L["type"]](L["mixer"], cfg.norm_eps,
                                   lambda k, p=p: get(p + "mix." + k), shard,
-                                  self._rope, dtype))
+                                  self._rope, self.dtype))
             if L.get("mlp"):
                 layer.norm2 = (get(p + "norm2"), get(p + "norm2.b"))
                 layer.ff = DenseGLU(shard.rows(get(p + "mlp.gate")),
                                     shard.rows(get(p + "mlp.up")),
                                     shard.cols(get(p + "mlp.down")))
             self.layers.append(layer)
-        self.ensure_positions(256)
-
-    @classmethod
-    def from_folder(cls, folder: str, config: dict, device: str = "cuda",
-                    dtype=torch.bfloat16, **kw) -> "LuzalornModel":
-        f = SafetensorsFile(os.path.join(folder, "model.safetensors"))
-        try:
-            return cls(LuzalornConfig.from_dict(config), device=device,
-                       dtype=dtype, weights=f, **kw)
-        finally:
-            f.close()
-
-    # ---- positions, cache --------------------------------------------------
-    def _rope(self, dims: int, base: float) -> RopeTable:
-        key = (dims, base)
-        if key not in self._ropes:
-            self._ropes[key] = RopeTable(dims, base, self.device)
-        return self._ropes[key]
-
-    def ensure_positions(self, n: int) -> None:
-        for r in self._ropes.values():
-            r.ensure(n)
-
-    def new_kv_cache(self, n_pages: int,
-                     state_slots: int | None = None) -> HybridCache:
-        kinds = [self.cfg.layers[r.layer] for r in self.runs]
-        return HybridCache(
-            n_pages, state_slots or 64,
-            [L["mixer"]["kv_rank"] for L in kinds
-             if L["type"] == "latent_attention"],
-            [MIXERS["retention"].state_shape(L["mixer"], self.shard)
-             for L in kinds if L["type"] == "retention"],
-            self.device, self.dtype)
 
     # ---- forward -----------------------------------------------------------
-    def _reduce(self, y: torch.Tensor) -> torch.Tensor:
-        if self.tp_size > 1:
-            import torch.distributed as dist
-            dist.all_reduce(y, group=self.tp_group)
-        return y
-
     def _forward(self, plan: StepPlan, kv: HybridCache,
                  rows: torch.Tensor | None,
                  trail: list | None = None) -> torch.Tensor:
-        """One step over all rows; logits of `rows` (None: every row).
-        trail collects the residual stream after every layer run."""
         eps = self.cfg.norm_eps
         res = torch.empty(plan.n_rows, self.cfg.hidden, dtype=torch.float32,
                           device=self.device)
@@ -296,38 +217,3 @@ class LuzalornModel:
         if rows is not None:
             res, y = res.index_select(0, rows), y.index_select(0, rows)
         return self.head(D.residual_norm(res, y, *self.final, eps))
-
-    @torch.no_grad()
-    def forward_decode(self, tokens: torch.Tensor, kv: HybridCache,
-                       block_table: torch.Tensor, seq_lens: torch.Tensor,
-                       positions: torch.Tensor,
-                       state_slots: torch.Tensor) -> torch.Tensor:
-        """tokens [B] i64 -> logits [B, vocab]; seq_lens INCLUDE the new
-        token.  Rows with seq_len 0 and slot -1 are padding."""
-        plan = StepPlan.decode(tokens, block_table, seq_lens, state_slots)
-        return self._forward(plan, kv, None)
-
-    @torch.no_grad()
-    def forward_prefill_batch(self, items, kv: HybridCache,
-                              want: list[list[int]] | None = None,
-                              trail: list | None = None) -> torch.Tensor:
-        """One step over entries (tokens [n] i64, seq_id, start): portions of
-        prompts of any length beside single tokens.  Returns the logits at
-        the places `want` of every entry (default: its last), in order."""
-        self.ensure_positions(max(int(s) + int(t.shape[0])
-                                  for t, _, s in items))
-        plan = StepPlan.build(items, kv)
-        first = {int(e): int(plan.offs[i]) for i, e in enumerate(plan.order)}
-        if want is None:
-            want = [[int(t.shape[0]) - 1] for t, _, _ in items]
-        rows = [first[e] + w for e, ws in enumerate(want) for w in ws]
-        # with nothing wanted the caches still have to advance: one row's
-        # logits are computed and dropped
-        idx = torch.tensor(rows or [0], dtype=torch.int64, device=self.device)
-        return self._forward(plan, kv, idx, trail)[:len(rows)]
-
-    @torch.no_grad()
-    def forward_prefill(self, tokens: torch.Tensor, kv: HybridCache,
-                        seq_id: int) -> torch.Tensor:
-        return self.forward_prefill_batch([(tokens, seq_id, 0)], kv)[0]
-

@@ -47,6 +47,8 @@ class Retention:
     """Linear attention with one fixed decay per head, rotated q and k, and
     a per-head rms norm gated by silu(W_g h)."""
 
+    storage = "state"            # which of the cache's lists a run indexes
+
     def __init__(self, m: dict, eps: float, get: Getter, shard: Shard,
                  rope: Callable[[int, float], RopeTable],
                  dtype: torch.dtype):
@@ -74,8 +76,8 @@ class Retention:
                 "g": (he, width), "o": (width, he)}
 
     @staticmethod
-    def state_shape(m: dict, shard: Shard) -> tuple[int, int, int]:
-        return shard.heads(m["heads"]), m["dim"], m["vdim"]
+    def cache(m: dict, shard: Shard) -> dict:
+        return {"state": (shard.heads(m["heads"]), m["dim"], m["vdim"])}
 
     def __call__(self, h: torch.Tensor, plan: StepPlan, kv,
                  run: int) -> torch.Tensor:
@@ -119,6 +121,7 @@ class LatentAttention:
     of the visible context by one GEMM, flash attention) for longer ones.
     """
 
+    storage = "latent"
     absorb_max = 16
 
     def __init__(self, m: dict, eps: float, get: Getter, shard: Shard,
@@ -155,6 +158,10 @@ class LatentAttention:
                 "uv": (H * m["vdim"], r), "sink": (H,),
                 "g": (H * m["vdim"], width), "o": (width, H * m["vdim"])}
 
+    @staticmethod
+    def cache(m: dict, shard: Shard) -> dict:
+        return {"latent": m["kv_rank"]}
+
     def __call__(self, h: torch.Tensor, plan: StepPlan, kv,
                  run: int) -> torch.Tensor:
         cache = kv.latents[run]
@@ -188,4 +195,214 @@ class LatentAttention:
         return self.out(y)
 
 
-MIXERS = {"retention": Retention, "latent_attention": LatentAttention}
+class ConvAttention:
+    """Branch: grouped-query attention whose q, k and v pass a short causal
+    convolution, then the rotation; per-head softmax sink, sigmoid output
+    gate.  Columns of the projection row: [q | k | v | gate].
+
+    Rows of portions of at most `rows_max` tokens are attended one by one (a
+    wave per share of a row's pages), longer portions block by block."""
+
+    rows_max = 16
+
+    def __init__(self, m: dict, out_scale: float, get: Getter, shard: Shard,
+                 rope: Callable[..., RopeTable], dtype: torch.dtype):
+        self.H, self.G = shard.heads(m["heads"]), shard.heads(m["kv_heads"])
+        self.D, self.E = m["dim"], m["vdim"]
+        if self.H % self.G:
+            raise ValueError("query heads do not divide over kv heads")
+        self.scale, self.out_scale = float(m["scale"]), float(out_scale)
+        rot = m.get("rot") or {"dims": 0, "base": 1.0}
+        self.rot = int(rot["dims"])
+        self.rope = rope(self.rot, float(rot["base"]), rot.get("scaling"))
+        self.channels = (self.H + self.G) * self.D + self.G * self.E
+        self.width = self.H * self.E
+        self.rows = torch.cat([shard.rows(get(n))
+                               for n in ("q", "k", "v", "g")])
+        self.out = shard.cols(get("o"))
+        self.filters = torch.cat(
+            [shard.rows(get(n + ".conv")) for n in ("q", "k", "v")]) \
+            .float().t().contiguous()
+        self.sink = shard.rows(get("sink")).float()
+        self.longest = None
+        if self.rows.is_cuda and dtype == torch.bfloat16 and \
+                D.gqa_mfma_ok(self.D, self.E):
+            self.longest = self.rows_max
+            self.block = D.gqa_portion_rows(self.D, self.E)
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> dict[str, tuple[int, ...]]:
+        q, k = m["heads"] * m["dim"], m["kv_heads"] * m["dim"]
+        v, o = m["kv_heads"] * m["vdim"], m["heads"] * m["vdim"]
+        return {"q": (q, width), "k": (k, width), "v": (v, width),
+                "q.conv": (q, m["conv"]), "k.conv": (k, m["conv"]),
+                "v.conv": (v, m["conv"]), "sink": (m["heads"],),
+                "g": (o, width), "o": (width, o)}
+
+    @staticmethod
+    def cache(m: dict, shard: Shard) -> dict:
+        g = shard.heads(m["kv_heads"])
+        c = (shard.heads(m["heads"]) + g) * m["dim"] + g * m["vdim"]
+        return {"kv": (g, m["dim"], m["vdim"]), "tail": (m["conv"] - 1, c)}
+
+    def __call__(self, x: torch.Tensor, plan: StepPlan, kv, run: int,
+                 tails: torch.Tensor, y: torch.Tensor) -> None:
+        c = self.channels
+        k, v = kv.keys[run], kv.values[run]
+        gate = x[:, c:c + self.width]
+        q = D.conv_qkv(x[:, :c], self.filters, tails, self.rope.cos,
+                       self.rope.sin, self.rot, plan.cache_slots, k, v,
+                       self.H, *plan.conv)
+        rows = plan.attn_rows(self.longest)
+        n = rows.n
+        if n:
+            D.gqa_rows(q[:n], k, v, rows.table, rows.item, rows.length,
+                       self.sink, gate[:n], y[:n], self.H, self.scale,
+                       self.out_scale)
+        if n < plan.n_rows:
+            p = plan.paged_portions(self.longest, self.block)
+            D.gqa_portions(q[n:], k, v, p.table, self.sink, gate[n:],
+                           p.qb_item, p.qb_t0, p.off, p.start, p.length,
+                           y[n:], self.H, self.scale, self.out_scale)
+
+
+class StateSpace:
+    """Branch: state-space duality (Mamba-2).  x, B and C pass a short causal
+    convolution and silu, the state decays by exp(-A dt) per head and token,
+    the gated read-out is rms-normed in equal parts.  Columns of the
+    projection row: [z | x | B | C | dt]."""
+
+    def __init__(self, m: dict, out_scale: float, eps: float, get: Getter,
+                 shard: Shard, dtype: torch.dtype):
+        self.H, self.P = shard.heads(m["heads"]), m["vdim"]
+        self.N, self.G = m["state"], shard.heads(m["groups"])
+        if self.H % self.G:
+            raise ValueError("heads do not divide over groups")
+        self.parts = shard.heads(m["norm_groups"])
+        self.eps = eps
+        self.width = self.H * self.P
+        if self.width % self.parts:
+            raise ValueError("inner width does not divide over norm groups")
+        inner, gn = m["heads"] * m["vdim"], m["groups"] * m["state"]
+        xbc = (inner, gn, gn)
+
+        def pieces(t, sizes):
+            return torch.cat([shard.rows(p) for p in t.split(sizes)])
+
+        self.rows = pieces(get("in"), (inner, *xbc, m["heads"]))
+        self.filters = pieces(get("conv"), xbc).float().t().contiguous()
+        self.bias = pieces(get("conv.b"), xbc).float()
+        self.dt_bias = shard.rows(get("dt_bias")).float()
+        self.A = torch.exp(shard.rows(get("A_log")).float())
+        self.skip = shard.rows(get("D")).float()
+        self.norm = shard.rows(get("norm")).float() * float(out_scale)
+        self.out = shard.cols(get("o"))
+        self.channels = self.filters.shape[1]
+        self.chunked = self.rows.is_cuda and dtype == torch.bfloat16 and \
+            D.ssd_chunked_ok(self.H, self.N, self.P, self.G)
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> dict[str, tuple[int, ...]]:
+        h, inner = m["heads"], m["heads"] * m["vdim"]
+        c = inner + 2 * m["groups"] * m["state"]
+        return {"in": (inner + c + h, width), "conv": (c, m["conv"]),
+                "conv.b": (c,), "dt_bias": (h,), "A_log": (h,), "D": (h,),
+                "norm": (inner,), "o": (width, inner)}
+
+    @staticmethod
+    def cache(m: dict, shard: Shard) -> dict:
+        h = shard.heads(m["heads"])
+        c = h * m["vdim"] + 2 * shard.heads(m["groups"]) * m["state"]
+        return {"state": (h, m["state"], m["vdim"]),
+                "tail": (m["conv"] - 1, c)}
+
+    def __call__(self, u: torch.Tensor, plan: StepPlan, kv, run: int,
+                 tails: torch.Tensor, y: torch.Tensor) -> None:
+        w, state = self.width, kv.states[run]
+        dt = w + self.channels
+        xbc = D.conv_silu(u[:, w:dt], self.filters, self.bias, tails,
+                          *plan.conv)
+        const = (self.A, self.dt_bias, self.skip, state, self.G)
+        n1 = plan.n_one
+        one = None
+        if n1:
+            one = D.ssd_decode(u[:n1], 0, dt, xbc[:n1], *const,
+                               plan.one_slots, plan.one_lens)
+        s = one
+        if n1 < plan.n_rows:
+            s = torch.empty(plan.n_rows, w, dtype=u.dtype, device=u.device)
+            if one is not None:
+                s[:n1] = one
+            args = (u[n1:], 0, dt, xbc[n1:], *const, plan.p_slots,
+                    plan.p_off, plan.p_start, plan.p_len)
+            if self.chunked:
+                D.ssd_chunked(*args, plan.chunk0, plan.chunk_item,
+                              plan.chunk_t0, s[n1:])
+            else:
+                D.ssd_seq(*args, s[n1:])
+        D.part_norm(s, self.norm, y, self.parts, self.eps)
+
+
+class Parallel:
+    """Attention and a state-space layer side by side on the same input:
+    left_scale * left + right_scale * right.  One GEMM projects for both, one
+    sums both: each branch writes its scaled columns of a common row."""
+
+    storage = "state"
+
+    def __init__(self, m: dict, eps: float, get: Getter, shard: Shard,
+                 rope, dtype: torch.dtype):
+        self.left = ConvAttention(m["left"], m["left_scale"],
+                                  lambda k: get("left." + k), shard, rope,
+                                  dtype)
+        self.right = StateSpace(m["right"], m["right_scale"], eps,
+                                lambda k: get("right." + k), shard, dtype)
+        # zero rows keep the branches' columns and the row stride aligned
+        rows, at = [], []
+        for part, unit in ((self.left, 8), (self.right, 16)):
+            at.append(sum(r.shape[0] for r in rows))
+            w = part.rows
+            del part.rows
+            rows += [w, w.new_zeros(-(at[-1] + w.shape[0]) % unit,
+                                    w.shape[1])]
+        self.at = at[1]
+        self.proj = Linear(torch.cat(rows))
+        self.out = Linear(torch.cat([self.left.out, self.right.out], 1))
+        del self.left.out, self.right.out
+
+    @staticmethod
+    def shapes(m: dict, width: int) -> dict[str, tuple[int, ...]]:
+        return {f"{side}.{k}": s for side, branch in
+                (("left", ConvAttention), ("right", StateSpace))
+                for k, s in branch.shapes(m[side], width).items()}
+
+    @staticmethod
+    def cache(m: dict, shard: Shard) -> dict:
+        a = ConvAttention.cache(m["left"], shard)
+        b = StateSpace.cache(m["right"], shard)
+        return {"state": b["state"], "kv": a["kv"],
+                "tails": (a["tail"], b["tail"])}
+
+    def __call__(self, h: torch.Tensor, plan: StepPlan, kv,
+                 run: int) -> torch.Tensor:
+        x = self.proj(h)
+        wl, wr = self.left.width, self.right.width
+        y = torch.empty(plan.n_rows, wl + wr, dtype=h.dtype, device=h.device)
+        tails = kv.tails[run]
+        self.left(x[:, :self.at], plan, kv, run, tails[0], y[:, :wl])
+        self.right(x[:, self.at:], plan, kv, run, tails[1], y[:, wl:])
+        return self.out(y)
+
+
+MIXERS = {"retention": Retention, "latent_attention": LatentAttention,
+          "parallel": Parallel}
+
+
+def cache_args(shapes: list[dict]) -> dict:
+    """Arguments of HybridCache for the runs of a model, each given by its
+    mixer's cache()."""
+    rec = [s for s in shapes if "state" in s]
+    return {"latent_ranks": [s["latent"] for s in shapes if "latent" in s],
+            "state_shapes": [s["state"] for s in rec],
+            "kv_shapes": [s.get("kv") for s in rec],
+            "tail_shapes": [s.get("tails", ()) for s in rec]}

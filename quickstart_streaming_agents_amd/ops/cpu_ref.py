@@ -106,23 +106,138 @@ def window_agg_ref(ts: torch.Tensor, key: torch.Tensor, value, t0: int,
 
 # ---- mixer decoders --------------------------------------------------------
 
-def residual_norm_ref(res, y, table, ids, vec, w, b, eps, init, layer):
+def residual_norm_ref(res, y, table, ids, vec, w, b, eps, init, layer, post,
+                      tscale):
     """In-place f32 residual update and its norm (dispatch.residual_norm)."""
+    like = y if w is None else w
     if init:
         res.zero_()
     if y is not None:
-        res.add_(y.float())
+        y = y.float()
+        if post is not None:
+            y = y / torch.sqrt(y.pow(2).mean(-1, keepdim=True) + eps) \
+                * post.float()
+        res.add_(y)
     if table is not None:
-        res.add_(table[ids].float())
+        res.add_(table[ids].float() * tscale)
     if vec is not None:
         res.add_(vec.float())
     x = res
+    if w is None:
+        return x.to(like.dtype, copy=True)
     if layer:
         x = x - x.mean(-1, keepdim=True)
     x = x / torch.sqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w.float()
     if b is not None:
         x = x + b.float()
     return x.to(w.dtype)
+
+
+def gated_act_ref(gate, factor, gelu):
+    g = gate.float()
+    g = torch.nn.functional.gelu(g, approximate="tanh") if gelu \
+        else torch.nn.functional.silu(g)
+    return (g * factor.float()).to(gate.dtype)
+
+
+def conv_portions(item, off, start, len_, slots):
+    """(slot, first row, first position, length) of a step's portions; without
+    `item`, one token per row at position start - 1 (0: row not in use)."""
+    if item is None:
+        return [(s, b, p - 1, 1) for b, (s, p) in
+                enumerate(zip(slots.tolist(), start.tolist()))
+                if s >= 0 and p > 0]
+    return list(zip(slots.tolist(), off.tolist(), start.tolist(),
+                    len_.tolist()))
+
+
+def short_conv_ref(x, w, tails, portions):
+    """Causal filters w [taps, C] over rows of x [T, C]; tails [slots,
+    taps - 1, C] carry the last inputs of every sequence.  f32 result."""
+    taps = w.shape[0]
+    y = torch.zeros(x.shape, dtype=torch.float32)
+    for slot, r0, p0, n in portions:
+        past = tails[slot].clone()
+        past[:max(0, taps - 1 - p0)] = 0        # before the sequence
+        u = torch.cat([past, x[r0:r0 + n]])
+        for j in range(taps):
+            y[r0:r0 + n] += w[j] * u[j:j + n].float()
+        tails[slot] = u[n:]
+    return y
+
+
+def conv_qkv_ref(x, w, tails, cos_t, sin_t, rot, cache_slots, kc, vc, heads,
+                 portions):
+    T, (_, G, _, D), E = x.shape[0], kc.shape, vc.shape[3]
+    y = short_conv_ref(x, w, tails, portions)
+    pos = torch.zeros(T, dtype=torch.int64)
+    live = torch.zeros(T, dtype=torch.bool)
+    for _, r0, p0, n in portions:
+        pos[r0:r0 + n] = torch.arange(p0, p0 + n)
+        live[r0:r0 + n] = True
+    qk = y[:, :(heads + G) * D].reshape(T, heads + G, D).clone()
+    if rot:
+        h = rot // 2
+        c, s = cos_t[pos][:, None], sin_t[pos][:, None]
+        a, b = qk[..., :h].clone(), qk[..., h:rot].clone()
+        qk[..., :h] = a * c - b * s
+        qk[..., h:rot] = b * c + a * s
+    v = y[:, (heads + G) * D:].reshape(T, G, E)
+    for t in range(T):
+        slot = int(cache_slots[t])
+        if live[t] and slot >= 0:
+            kc[slot // 64, :, slot % 64] = qk[t, heads:].to(kc.dtype)
+            vc[slot // 64, :, slot % 64] = v[t].to(vc.dtype)
+    return qk[:, :heads].reshape(T, heads * D).to(x.dtype)
+
+
+def gqa_rows_ref(q, kc, vc, block_table, row_item, row_len, sink, gate, out,
+                 heads, scale, out_scale):
+    R, (_, G, _, D), E = q.shape[0], kc.shape, vc.shape[3]
+    for r in range(R):
+        n = int(row_len[r])
+        if n <= 0:
+            out[r] = 0
+            continue
+        pos = torch.arange(n)
+        page = block_table[int(row_item[r]) if row_item is not None
+                           else r].long()[pos // 64]
+        k = kc[page, :, pos % 64].float().transpose(0, 1)      # [G, n, D]
+        v = vc[page, :, pos % 64].float().transpose(0, 1)
+        s = torch.matmul(q[r].float().view(G, heads // G, D),
+                         k.transpose(1, 2)) * scale
+        if sink is not None:
+            s = torch.cat([s, sink.view(G, -1, 1)], -1)
+        o = torch.matmul(torch.softmax(s, -1)[..., :n], v).reshape(-1)
+        if gate is not None:
+            o = o * torch.sigmoid(gate[r].float())
+        out[r] = (o * out_scale).to(out.dtype)
+
+
+def ssd_ref(u, zoff, dtoff, xbc, A, dt_bias, D, state, groups, portions, out):
+    """portions: (slot, first row, first position, length); state and the
+    portions' rows of out are written."""
+    _, H, N, P = state.shape
+    inner = H * P
+    for slot, r0, p0, n in portions:
+        rows = xbc[r0:r0 + n].float()
+        x = rows[:, :inner].reshape(n, H, P)
+        B, C = (t.reshape(n, groups, N).repeat_interleave(H // groups, 1)
+                for t in rows[:, inner:].chunk(2, 1))
+        z = u[r0:r0 + n, zoff:zoff + inner].float()
+        dt = torch.nn.functional.softplus(
+            u[r0:r0 + n, dtoff:dtoff + H].float() + dt_bias)
+        S = state[slot]
+        if p0 == 0:
+            S.zero_()
+        y = torch.empty(n, H, P)
+        for t in range(n):
+            S.mul_(torch.exp(-A * dt[t])[:, None, None]).add_(
+                (B[t] * dt[t][:, None])[:, :, None] * x[t][:, None, :])
+            y[t] = torch.matmul(C[t][:, None, :], S).squeeze(1) \
+                + D[:, None] * x[t]
+        out[r0:r0 + n] = (y.reshape(n, inner)
+                          * torch.nn.functional.silu(z)).to(out.dtype)
 
 
 def latent_rows_ref(qa, cache, block_table, row_item, row_len, sink, window,

@@ -229,25 +229,42 @@ def skinny_linear_fp8(x: torch.Tensor, qf: torch.Tensor,
 # ops/cpu_ref.py.
 
 def residual_norm(res: torch.Tensor, y: torch.Tensor | None,
-                  w: torch.Tensor, b: torch.Tensor | None, eps: float, *,
-                  table: torch.Tensor | None = None,
+                  w: torch.Tensor | None, b: torch.Tensor | None,
+                  eps: float, *, table: torch.Tensor | None = None,
                   ids: torch.Tensor | None = None,
                   vec: torch.Tensor | None = None, init: bool = False,
-                  layer: bool = True) -> torch.Tensor:
-    """res (f32) <- (0 if init else res) + y + table[ids] + vec, in place;
-    returns the layer norm (layer=True) or rms norm of it, times w, plus b."""
+                  layer: bool = True, post: torch.Tensor | None = None,
+                  tscale: float = 1.0) -> torch.Tensor:
+    """res (f32) <- (0 if init else res) + y + tscale * table[ids] + vec, in
+    place; returns the layer norm (layer=True) or rms norm of it, times w,
+    plus b, or without w the residual itself.  With `post`, y enters as its
+    own rms norm times post."""
     if _cuda(res):
         return lm_ext().residual_norm(res, y, table, ids, vec, w, b, eps,
-                                      init, layer)
+                                      init, layer, post, tscale)
     from .cpu_ref import residual_norm_ref
-    return residual_norm_ref(res, y, table, ids, vec, w, b, eps, init, layer)
+    return residual_norm_ref(res, y, table, ids, vec, w, b, eps, init, layer,
+                             post, tscale)
 
 
-def glu(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
-    """silu(gate) * up for any width and storage type."""
+def glu(gate: torch.Tensor, up: torch.Tensor,
+        act: str = "silu") -> torch.Tensor:
+    """act(gate) * up for any width and storage type; act: silu or gelu (its
+    tanh form)."""
     if _cuda(gate):
-        return lm_ext().glu(gate, up)
-    return (torch.nn.functional.silu(gate.float()) * up.float()).to(gate.dtype)
+        return lm_ext().glu(gate, up, act == "gelu")
+    from .cpu_ref import gated_act_ref
+    return gated_act_ref(gate, up, act == "gelu")
+
+
+def glu_table(gate: torch.Tensor, table: torch.Tensor, ids: torch.Tensor,
+              col0: int, act: str = "gelu") -> torch.Tensor:
+    """act(gate [T, n]) * table[ids, col0 : col0 + n]."""
+    if _cuda(gate):
+        return lm_ext().glu_table(gate, table, ids, col0, act == "gelu")
+    from .cpu_ref import gated_act_ref
+    return gated_act_ref(gate, table[ids, col0:col0 + gate.shape[1]],
+                         act == "gelu")
 
 
 def argmax_rows(x: torch.Tensor) -> torch.Tensor:
@@ -369,6 +386,121 @@ def retention_chunked(x, cos_t, sin_t, log2_decay, state, slots, off, start,
     lm_ext().retention_chunked(x, cos_t, sin_t, log2_decay, state, slots,
                                off, start, len_, positions, chunk0,
                                chunk_item, chunk_t0, out, rot, kscale, eps)
+
+
+# A step's rows for the short convolutions are (item, t0, off, start, len,
+# slots): portions in chunks of 16 rows, or, with item None, one token per row
+# at position start - 1 (layers.StepPlan.conv).
+
+def conv_qkv(x, filters, tails, cos_t, sin_t, rot: int, cache_slots, kc, vc,
+             heads: int, item, t0, off, start, len_, slots) -> torch.Tensor:
+    """x columns [q | k | v] through their causal filters [taps, C], q and k
+    rotated; returns q, writes k and v to their pages [P, G, 64, .] at
+    cache_slots.  tails [slots, taps - 1, C] hold the last inputs."""
+    if _cuda(x):
+        return lm_ext().conv_qkv(x, filters, tails, cos_t, sin_t, rot,
+                                 cache_slots, kc, vc, heads, item, t0, off,
+                                 start, len_, slots)
+    from .cpu_ref import conv_portions, conv_qkv_ref
+    return conv_qkv_ref(x, filters, tails, cos_t, sin_t, rot, cache_slots,
+                        kc, vc, heads,
+                        conv_portions(item, off, start, len_, slots))
+
+
+def conv_silu(x, filters, bias, tails, item, t0, off, start, len_,
+              slots) -> torch.Tensor:
+    """silu(causal filters over x + bias), dense [T, C]."""
+    if _cuda(x):
+        return lm_ext().conv_silu(x, filters, bias, tails, item, t0, off,
+                                  start, len_, slots)
+    from .cpu_ref import conv_portions, short_conv_ref
+    y = short_conv_ref(x, filters, tails,
+                       conv_portions(item, off, start, len_, slots))
+    return torch.nn.functional.silu(y + bias).to(x.dtype)
+
+
+def gqa_rows(q, kc, vc, block_table, row_item, row_len, sink, gate, out,
+             heads: int, scale: float, out_scale: float = 1.0) -> None:
+    """Rows of q [R, heads*D] at positions row_len - 1 over the paged keys
+    and values of sequence row_item (their own index without it): softmax with
+    sink, times sigmoid(gate) and out_scale, to rows of out."""
+    if _cuda(q):
+        lm_ext().gqa_rows(q, kc, vc, block_table, row_item, row_len, sink,
+                          gate, out, heads, scale, out_scale)
+        return
+    from .cpu_ref import gqa_rows_ref
+    gqa_rows_ref(q, kc, vc, block_table, row_item, row_len, sink, gate, out,
+                 heads, scale, out_scale)
+
+
+def gqa_mfma_ok(d: int, e: int) -> bool:
+    return lm_ext().gqa_mfma_ok(d, e)
+
+
+def gqa_portion_rows(d: int, e: int) -> int:
+    return lm_ext().gqa_portion_rows(d, e)
+
+
+def gqa_portions(q, kc, vc, block_table, sink, gate, qb_item, qb_t0, off,
+                 start, len_, out, heads: int, scale: float,
+                 out_scale: float = 1.0) -> None:
+    """The same for whole portions, flash attention (GPU, bf16)."""
+    lm_ext().gqa_portions(q, kc, vc, block_table, sink, gate, qb_item, qb_t0,
+                          off, start, len_, out, heads, scale, out_scale)
+
+
+def ssd_decode(u, zoff: int, dtoff: int, xbc, A, dt_bias, D, state,
+               groups: int, slots, seq_lens) -> torch.Tensor:
+    """One token per row of a state-space layer: z and raw dt are columns of
+    u, x | B | C are xbc, state [slots, H, N, P] f32 updated in place.
+    Returns (S^T C + D x) * silu(z).  Rows with seq_len 0 or slot -1 are not
+    in use."""
+    if _cuda(u):
+        return lm_ext().ssd_decode(u, zoff, dtoff, xbc, A, dt_bias, D, state,
+                                   groups, slots, seq_lens)
+    from .cpu_ref import conv_portions, ssd_ref
+    out = torch.zeros(u.shape[0], state.shape[1] * state.shape[3],
+                      dtype=u.dtype)
+    ssd_ref(u, zoff, dtoff, xbc, A, dt_bias, D, state, groups,
+            conv_portions(None, None, seq_lens, None, slots), out)
+    return out
+
+
+def ssd_seq(u, zoff: int, dtoff: int, xbc, A, dt_bias, D, state, groups: int,
+            slots, off, start, len_, out) -> None:
+    """Portions of several tokens, token by token (any size and type)."""
+    if _cuda(u):
+        lm_ext().ssd_seq(u, zoff, dtoff, xbc, A, dt_bias, D, state, groups,
+                         slots, off, start, len_, out)
+        return
+    from .cpu_ref import ssd_ref
+    ssd_ref(u, zoff, dtoff, xbc, A, dt_bias, D, state, groups,
+            list(zip(slots.tolist(), off.tolist(), start.tolist(),
+                     len_.tolist())), out)
+
+
+def ssd_chunked_ok(h: int, n: int, p: int, groups: int) -> bool:
+    return lm_ext().ssd_chunked_ok(h, n, p, groups)
+
+
+def ssd_chunked(u, zoff: int, dtoff: int, xbc, A, dt_bias, D, state,
+                groups: int, slots, off, start, len_, chunk0, chunk_item,
+                chunk_t0, out) -> None:
+    """Portions in chunks of 64 tokens on the matrix cores (GPU, bf16)."""
+    lm_ext().ssd_chunked(u, zoff, dtoff, xbc, A, dt_bias, D, state, groups,
+                         slots, off, start, len_, chunk0, chunk_item,
+                         chunk_t0, out)
+
+
+def part_norm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor,
+              parts: int, eps: float) -> None:
+    """out <- rms norm of `parts` equal parts of every row of x, times w."""
+    if _cuda(x):
+        lm_ext().part_norm(x, w, out, parts, eps)
+        return
+    y = x.float().view(x.shape[0], parts, -1)
+    y = y / torch.sqrt(y.pow(2).mean(-1, keepdim=True) + eps)
+    out.copy_((y.reshape(x.shape) * w).to(out.dtype))
 
 
 # ---- retrieval / streaming ------------------------------------------------

@@ -4,21 +4,25 @@
 
 // ---------------------------------------------------------------------------
 // Residual update and norm of one row, everything in f32:
-//   r   = (init ? 0 : res) + y + table[ids[row]] + vec      (each optional)
+//   r   = (init ? 0 : res) + p + tscale * table[ids[row]] + vec
+//         (p, table, vec optional); p = y, or with POST the branch's own norm
+//         y / sqrt(mean y^2 + eps) * post
 //   res = r
 //   out = norm(r) * w + b      LAYER: (r - mean)/sqrt(var + eps), var the
 //                              mean squared deviation; else r/sqrt(mean r^2
-//                              + eps).  b optional.
+//                              + eps).  b optional; without w, out = r.
 // The row stays in registers between the passes up to CACHED groups per
 // thread; wider rows re-read the residual this thread wrote itself.
 // ---------------------------------------------------------------------------
-template <typename T, int VEC, bool LAYER>
+template <typename T, int VEC, bool LAYER, bool POST>
 __global__ void __launch_bounds__(1024)
 qsa_residual_norm(float* __restrict__ res, const T* __restrict__ y,
-                  long long ystride, const T* __restrict__ table,
-                  const long long* __restrict__ ids, const T* __restrict__ vec,
-                  const T* __restrict__ w, const T* __restrict__ b,
-                  T* __restrict__ out, int W, int vocab, float eps, int init) {
+                  long long ystride, const T* __restrict__ post,
+                  const T* __restrict__ table,
+                  const long long* __restrict__ ids, float tscale,
+                  const T* __restrict__ vec, const T* __restrict__ w,
+                  const T* __restrict__ b, T* __restrict__ out, int W,
+                  int vocab, float eps, int init) {
   constexpr int CACHED = 8;
   __shared__ float scratch[16];
   const long long row = blockIdx.x;
@@ -33,24 +37,56 @@ qsa_residual_norm(float* __restrict__ res, const T* __restrict__ y,
   const int step = blockDim.x * VEC;
   const int i0 = threadIdx.x * VEC;
   float cache[CACHED][VEC];
+  float pinv = 1.f;
+  if (POST) {
+    float ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < CACHED; ++c) {
+      const int i = i0 + c * step;
+      if (i < W) {
+        ldv<T, VEC>(yr + i, cache[c]);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) ss = fmaf(cache[c][j], cache[c][j], ss);
+      }
+    }
+    for (int i = i0 + CACHED * step; i < W; i += step) {
+      float v[VEC];
+      ldv<T, VEC>(yr + i, v);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) ss = fmaf(v[j], v[j], ss);
+    }
+    pinv = 1.f / sqrtf(block_reduce_sum(ss, scratch) / (float)W + eps);
+  }
   float sum = 0.f;
+  // v: on entry, with POST, the branch's output
   auto load_row = [&](int i, float* v) {
     float t[VEC];
-    if (init) {
+    if (POST) {
+      ldv<T, VEC>(post + i, t);
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) v[j] = 0.f;
+      for (int j = 0; j < VEC; ++j) v[j] *= pinv * t[j];
+      if (!init) {
+        ldv<float, VEC>(rr + i, t);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) v[j] += t[j];
+      }
     } else {
-      ldv<float, VEC>(rr + i, v);
-    }
-    if (yr) {
-      ldv<T, VEC>(yr + i, t);
+      if (init) {
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) v[j] += t[j];
+        for (int j = 0; j < VEC; ++j) v[j] = 0.f;
+      } else {
+        ldv<float, VEC>(rr + i, v);
+      }
+      if (yr) {
+        ldv<T, VEC>(yr + i, t);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) v[j] += t[j];
+      }
     }
     if (er) {
       ldv<T, VEC>(er + i, t);
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) v[j] += t[j];
+      for (int j = 0; j < VEC; ++j) v[j] = fmaf(tscale, t[j], v[j]);
     }
     if (vec) {
       ldv<T, VEC>(vec + i, t);
@@ -71,9 +107,22 @@ qsa_residual_norm(float* __restrict__ res, const T* __restrict__ y,
   }
   for (int i = i0 + CACHED * step; i < W; i += step) {
     float v[VEC];
+    if (POST) ldv<T, VEC>(yr + i, v);
     load_row(i, v);
 #pragma unroll
     for (int j = 0; j < VEC; ++j) sum += LAYER ? v[j] : v[j] * v[j];
+  }
+  T* orow = out + row * W;
+  if (!w) {                                         // the residual itself
+#pragma unroll
+    for (int c = 0; c < CACHED; ++c)
+      if (i0 + c * step < W) stv<T, VEC>(orow + i0 + c * step, cache[c]);
+    for (int i = i0 + CACHED * step; i < W; i += step) {
+      float v[VEC];
+      ldv<float, VEC>(rr + i, v);
+      stv<T, VEC>(orow + i, v);
+    }
+    return;
   }
   sum = block_reduce_sum(sum, scratch);
   float mean = 0.f, ms = sum / (float)W;
@@ -101,7 +150,6 @@ qsa_residual_norm(float* __restrict__ res, const T* __restrict__ y,
     ms = block_reduce_sum(dev, scratch) / (float)W;
   }
   const float inv = 1.f / sqrtf(ms + eps);
-  T* orow = out + row * W;
   auto emit = [&](int i, const float* v) {
     float t[VEC], o[VEC];
     ldv<T, VEC>(w + i, t);
@@ -124,9 +172,10 @@ qsa_residual_norm(float* __restrict__ res, const T* __restrict__ y,
   }
 }
 
-template <typename T, int VEC, bool LAYER>
+template <typename T, int VEC, bool LAYER, bool POST>
 static void residual_norm_go(float* res, const void* y, long long ystride,
-                             const void* table, const long long* ids,
+                             const void* post, const void* table,
+                             const long long* ids, float tscale,
                              const void* vec, const void* w, const void* b,
                              void* out, long long rows, int W, int vocab,
                              float eps, int init, hipStream_t st) {
@@ -134,67 +183,97 @@ static void residual_norm_go(float* res, const void* y, long long ystride,
   // few rows: wide blocks, one round of loads; many rows: narrow ones
   const int most = rows <= 256 ? 1024 : 256;
   threads = threads > most ? most : threads;
-  hipLaunchKernelGGL((qsa_residual_norm<T, VEC, LAYER>), dim3((unsigned)rows),
-                     dim3(threads), 0, st, res, (const T*)y, ystride,
-                     (const T*)table, ids, (const T*)vec, (const T*)w,
-                     (const T*)b, (T*)out, W, vocab, eps, init);
+  hipLaunchKernelGGL((qsa_residual_norm<T, VEC, LAYER, POST>),
+                     dim3((unsigned)rows), dim3(threads), 0, st, res,
+                     (const T*)y, ystride, (const T*)post, (const T*)table,
+                     ids, tscale, (const T*)vec, (const T*)w, (const T*)b,
+                     (T*)out, W, vocab, eps, init);
 }
 
 extern "C" void qsa_residual_norm_launch(
-    float* res, const void* y, long long ystride, const void* table,
-    const long long* ids, const void* vec, const void* w, const void* b,
-    void* out, long long rows, int W, int vocab, float eps, int init,
-    int layer, int f32, int vec4, hipStream_t st) {
-#define QSA_RN(T, V, L)                                                      \
-  residual_norm_go<T, V, L>(res, y, ystride, table, ids, vec, w, b, out,     \
-                            rows, W, vocab, eps, init, st)
+    float* res, const void* y, long long ystride, const void* post,
+    const void* table, const long long* ids, float tscale, const void* vec,
+    const void* w, const void* b, void* out, long long rows, int W, int vocab,
+    float eps, int init, int layer, int f32, int vec4, hipStream_t st) {
+#define QSA_RN(T, V, L, P)                                                    \
+  residual_norm_go<T, V, L, P>(res, y, ystride, post, table, ids, tscale,     \
+                               vec, w, b, out, rows, W, vocab, eps, init, st)
+#define QSA_RN_L(T, V)                                                        \
+  if (layer) { if (post) QSA_RN(T, V, true, true);                            \
+               else QSA_RN(T, V, true, false); }                              \
+  else { if (post) QSA_RN(T, V, false, true);                                 \
+         else QSA_RN(T, V, false, false); }
   if (f32) {
-    if (vec4) { if (layer) QSA_RN(float, 4, true); else QSA_RN(float, 4, false); }
-    else      { if (layer) QSA_RN(float, 1, true); else QSA_RN(float, 1, false); }
+    if (vec4) { QSA_RN_L(float, 4) } else { QSA_RN_L(float, 1) }
   } else {
-    if (vec4) { if (layer) QSA_RN(bf16_t, 4, true); else QSA_RN(bf16_t, 4, false); }
-    else      { if (layer) QSA_RN(bf16_t, 1, true); else QSA_RN(bf16_t, 1, false); }
+    if (vec4) { QSA_RN_L(bf16_t, 4) } else { QSA_RN_L(bf16_t, 1) }
   }
+#undef QSA_RN_L
 #undef QSA_RN
 }
 
 // ---------------------------------------------------------------------------
-// Gated linear unit: out = silu(gate) * up over [rows, cols] strided halves.
+// Gated activations.  The factor is the other half of a projection (a gated
+// linear unit) or a slice of the token's row of a table:
+//   out[r, c] = act(gate[r, c]) * up[r, c]
+//   out[r, c] = act(gate[r, c]) * table[ids[r], col0 + c]
+// act: silu, or the tanh form of gelu, z / (1 + exp(-2 sqrt(2/pi)
+// (z + 0.044715 z^3))).
 // ---------------------------------------------------------------------------
-template <typename T, int VEC>
+#define QSA_ACT_SILU 0
+#define QSA_ACT_GELU 1
+
+template <bool EXACT, int ACT>
+__device__ __forceinline__ float act_f(float z) {
+  const float a = ACT == QSA_ACT_SILU
+      ? z : 1.5957691216057308f * fmaf(0.044715f * z * z, z, z);
+  return z / (1.f + (EXACT ? expf(-a) : __expf(-a)));
+}
+
+template <typename T, int VEC, int ACT>
 __global__ void __launch_bounds__(256)
 qsa_glu(const T* __restrict__ gate, const T* __restrict__ up,
-        T* __restrict__ out, long long rows, long long cols,
-        long long stride) {
+        const long long* __restrict__ ids, T* __restrict__ out,
+        long long rows, long long cols, long long stride, long long ustride,
+        long long vocab) {
   const long long groups = cols / VEC;
   const long long n = rows * groups;
   for (long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x; i < n;
        i += (long long)gridDim.x * blockDim.x) {
     const long long r = i / groups, c = (i % groups) * VEC;
+    long long ur = r;
+    if (ids) {
+      ur = ids[r];
+      ur = ur < 0 ? 0 : (ur >= vocab ? vocab - 1 : ur);
+    }
     float g[VEC], u[VEC];
     ldv<T, VEC>(gate + r * stride + c, g);
-    ldv<T, VEC>(up + r * stride + c, u);
+    ldv<T, VEC>(up + ur * ustride + c, u);
 #pragma unroll
     for (int j = 0; j < VEC; ++j)
-      g[j] = (sizeof(T) == 4 ? silu_f(g[j]) : g[j] / (1.f + __expf(-g[j]))) *
-             u[j];
+      g[j] = act_f<sizeof(T) == 4, ACT>(g[j]) * u[j];
     stv<T, VEC>(out + r * cols + c, g);
   }
 }
 
-extern "C" void qsa_glu_launch(const void* gate, const void* up, void* out,
+extern "C" void qsa_glu_launch(const void* gate, const void* up,
+                               const long long* ids, void* out,
                                long long rows, long long cols,
-                               long long stride, int f32, int vec,
+                               long long stride, long long ustride,
+                               long long vocab, int gelu, int f32, int vec,
                                hipStream_t st) {
   const long long n = rows * (cols / (vec ? 8 : 1));
   const long long want = (n + 255) / 256;
   dim3 grid((unsigned)(want < 1 ? 1 : (want > 16384 ? 16384 : want)));
-#define QSA_GLU(T, V)                                                      \
-  hipLaunchKernelGGL((qsa_glu<T, V>), grid, dim3(256), 0, st,              \
-                     (const T*)gate, (const T*)up, (T*)out, rows, cols,    \
-                     stride)
-  if (f32) { if (vec) QSA_GLU(float, 8); else QSA_GLU(float, 1); }
-  else     { if (vec) QSA_GLU(bf16_t, 8); else QSA_GLU(bf16_t, 1); }
+#define QSA_GLU(T, V, A)                                                   \
+  hipLaunchKernelGGL((qsa_glu<T, V, A>), grid, dim3(256), 0, st,           \
+                     (const T*)gate, (const T*)up, ids, (T*)out, rows,     \
+                     cols, stride, ustride, vocab)
+#define QSA_GLU_A(T, V)                                                    \
+  if (gelu) QSA_GLU(T, V, QSA_ACT_GELU); else QSA_GLU(T, V, QSA_ACT_SILU)
+  if (f32) { if (vec) { QSA_GLU_A(float, 8); } else { QSA_GLU_A(float, 1); } }
+  else     { if (vec) { QSA_GLU_A(bf16_t, 8); } else { QSA_GLU_A(bf16_t, 1); } }
+#undef QSA_GLU_A
 #undef QSA_GLU
 }
 

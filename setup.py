@@ -38,7 +38,8 @@ MODULES = {
                 "hash_join.hip", "gemm_fp8_batch.hip", "topk_cosine.hip",
                 "streaming.hip"],
     "qsa_lm_hip": ["lm_ops.cpp", "lm_elementwise.hip", "retention.hip",
-                   "latent_attn.hip", "skinny_gemm.hip"],
+                   "latent_attn.hip", "short_conv.hip", "gqa_attn.hip", "ssd.hip",
+                   "skinny_gemm.hip"],
 }
 
 
