@@ -55,10 +55,11 @@ def parse_args():
                         "scheduler")
     p.add_argument("--workload", default="lab1",
                    choices=("lab1", "luzalorn", "luzalorn-kernels",
-                            "luzalorn-models"),
-                   help="lab1: the headline benchmark (default); luzalorn: "
-                        "prefill/decode throughput and kernel rooflines of "
-                        "that design beside the Llama decoder")
+                            "luzalorn-models", "lunulix", "lunulix-kernels",
+                            "lunulix-models"),
+                   help="lab1: the headline benchmark (default); a mixer "
+                        "design: its prefill/decode throughput and kernel "
+                        "rooflines beside the framework's other decoders")
     p.add_argument("--stub-llm", action="store_true",
                    help="CPU contract check: stub LLM instead of the GPU engine")
     return p.parse_args()
@@ -68,7 +69,7 @@ def main():
     args = parse_args()
     if args.workload != "lab1":
         from quickstart_streaming_agents_amd.models import bench as models_bench
-        models_bench.main(args.workload.partition("-")[2] or "all")
+        models_bench.main(args.workload)
         return
     import torch
 

@@ -1,10 +1,10 @@
-"""Throughput of the Luzalorn design beside the Llama decoder at equal width,
+"""Throughput of the mixer decoders beside the Llama decoder at equal width,
 feed-forward and depth, and kernel by kernel against the roofline.
 
-    python bench.py --workload luzalorn
+    python bench.py --workload luzalorn     (or lunulix)
 
 Random weights, synthetic tokens.  One JSON line per measurement:
-  {"kind": "model", ...}   prefill and decode tokens/s of both models
+  {"kind": "model", ...}   prefill and decode tokens/s of the models
   {"kind": "kernel", ...}  time of a kernel (launched back to back inside a
                            graph, operands rotated so that they do not stay
                            in cache), its roofline time max(bytes / 8 TB/s,
@@ -211,10 +211,13 @@ def bench_kernels(reps: int = 8) -> None:
             shape=[n_seq, n, H, KVH, Dm])
 
 
-def _models(width: int, ff: int, layers: int):
+def _models(width: int, ff: int, layers: int, names: tuple):
+    """(name, class, configuration) of decoders of equal size."""
     from .llama import LlamaConfig, LlamaModel
+    from .lunulix import LunulixConfig, LunulixModel
     from .luzalorn import LuzalornConfig, LuzalornModel
     heads = width // 128
+    mlp = {"kind": "dense", "ff": ff}
     ret = {"type": "retention", "mixer": {
         "heads": heads // 2, "dim": 128, "vdim": 256,
         "decay": [1 - 2.0 ** (-5 - i % 6) for i in range(heads // 2)],
@@ -222,21 +225,33 @@ def _models(width: int, ff: int, layers: int):
     lat = {"type": "latent_attention", "mixer": {
         "heads": heads, "dim": 128, "vdim": 128, "q_rank": width * 3 // 8,
         "kv_rank": 512, "scale": 128 ** -0.5, "mask": {"size": 4096}}}
-    mlp = {"kind": "dense", "ff": ff}
-    lz = LuzalornConfig(
-        layers=[dict(lat if i % 4 == 3 else ret, mlp=mlp)
-                for i in range(layers)], vocab_size=32_000, hidden=width)
-    ll = LlamaConfig(name="bench", vocab_size=32_000, hidden=width,
-                     n_layers=layers, n_q_heads=heads, n_kv_heads=8,
-                     d_head=128, ffn=ff, max_pos=16_384)
-    yield "luzalorn", LuzalornModel, lz
-    yield "llama", LlamaModel, ll
+    par = {"type": "parallel", "mixer": {
+        "left": {"heads": heads, "kv_heads": 8, "dim": 128, "vdim": 128,
+                 "conv": 4, "scale": 128 ** -0.5,
+                 "rot": {"dims": 128, "base": 5e5}}, "left_scale": 0.7,
+        "right": {"heads": width // 64, "vdim": 64, "state": 128,
+                  "groups": 8, "conv": 4, "norm_groups": 8},
+        "right_scale": 0.7}}
+    found = {
+        "luzalorn": (LuzalornModel, LuzalornConfig(
+            layers=[dict(lat if i % 4 == 3 else ret, mlp=mlp)
+                    for i in range(layers)], vocab_size=32_000,
+            hidden=width)),
+        "lunulix": (LunulixModel, LunulixConfig(
+            layers=[dict(par, mlp=mlp)] * layers, vocab_size=32_000,
+            hidden=width, side_dim=width // 16)),
+        "llama": (LlamaModel, LlamaConfig(
+            name="bench", vocab_size=32_000, hidden=width, n_layers=layers,
+            n_q_heads=heads, n_kv_heads=8, d_head=128, ffn=ff,
+            max_pos=16_384))}
+    for name in names:
+        yield name, *found[name]
 
 
-def bench_models(layers: int = 8) -> None:
+def bench_models(names: tuple, layers: int = 8) -> None:
     from .serve import Engine
     for width, ff in ((2048, 8192), (4096, 14_336)):
-        for name, cls, cfg in _models(width, ff, layers):
+        for name, cls, cfg in _models(width, ff, layers, names):
             model = cls(cfg, device="cuda:0")
             for n_seq, n in ((1, 8192), (16, 1024)):
                 kv = model.new_kv_cache(n_seq * n // 64, state_slots=n_seq)
@@ -281,9 +296,16 @@ def bench_models(layers: int = 8) -> None:
             torch.cuda.empty_cache()
 
 
-def main(part: str = "all") -> None:
-    if part in ("all", "kernels"):
+def main(workload: str) -> None:
+    """workload: <design>[-kernels | -models]"""
+    design, _, part = workload.partition("-")
+    if part in ("", "kernels"):
         with torch.no_grad():
-            bench_kernels()
-    if part in ("all", "models"):
-        bench_models()
+            if design == "lunulix":
+                from .bench_lunulix import bench_kernels as kernels
+                kernels()
+            else:
+                bench_kernels()
+    if part in ("", "models"):
+        bench_models((design, "llama") if design == "luzalorn" else
+                     (design, "luzalorn", "llama"))

@@ -76,9 +76,9 @@ CONFIGS = {
                         right(2, 24, 32, 2, 4, 4), 44)),
     # one of everything: no taps beyond the current token, nothing rotated
     "ones": model(96, 64, 48,
-                  par(left(1, 1, 32, 16, 1, 0, 0.4), right(1, 32, 16, 1, 1,
+                  par(left(1, 1, 32, 16, 1, 0, 0.2), right(1, 32, 16, 1, 1,
                                                            1), 64, 1.0, 1.0),
-                  par(left(1, 1, 16, 32, 2, 2, 1.0), right(1, 8, 8, 1, 2, 1),
+                  par(left(1, 1, 16, 32, 2, 2, 0.5), right(1, 8, 8, 1, 2, 1),
                       72, 1.0, 1.0), scale=1.0),
     # wide heads and states, more query heads per key head than one tile has
     "wide": model(200, 256, 40,
@@ -137,12 +137,15 @@ class Case(MixerCase):
         if self.dtype != torch.bfloat16 or toks is None:
             return plain
         if toks not in self._shaken:
-            g = torch.Generator().manual_seed(1)
-            w = {k: t.double() * (1 + 2 ** -8 * torch.randn(
-                t.shape, generator=g)) for k, t in self.weights.items()}
-            self._shaken[toks] = row_errors(
-                self.forward(self.raw, w, list(toks))[0], want)
-        return torch.maximum(plain, 1.5 * self._shaken[toks])
+            err = []
+            for seed in range(3):
+                g = torch.Generator().manual_seed(seed)
+                w = {k: t.double() * (1 + 2 ** -8 * torch.randn(
+                    t.shape, generator=g)) for k, t in self.weights.items()}
+                err.append(row_errors(self.forward(self.raw, w,
+                                                   list(toks))[0], want))
+            self._shaken[toks] = torch.stack(err).max(0).values
+        return torch.maximum(plain, 2 * self._shaken[toks])
 
 
 # ---- keys far away ----------------------------------------------------------
