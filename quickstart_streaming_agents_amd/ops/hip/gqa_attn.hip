@@ -18,6 +18,11 @@
 #define NEG_BIG (-3.0e38f)
 #define LOG2E 1.4426950408889634f
 
+// 2^x by the hardware instruction; what would be denormal becomes zero
+__device__ __forceinline__ float exp2_hw(float x) {
+  return __builtin_amdgcn_exp2f(x);
+}
+
 template <typename T>
 __global__ void __launch_bounds__(256)
 qsa_gqa_rows(const T* __restrict__ q, const T* __restrict__ kc,
@@ -221,7 +226,8 @@ qsa_gqa_rows_mfma(const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc,
       mx = fmaxf(mx, __shfl_xor(mx, 16, QSA_WAVE));
       mx = fmaxf(mx, __shfl_xor(mx, 32, QSA_WAVE));
       const float mn = fmaxf(m, mx);
-      const float alpha = m > NEG_BIG ? exp2f(m - mn) : 0.f;
+      const float alpha = exp2_hw(m - mn);        // a step sees a key: mn is
+                                                  // finite, masked terms 0
       m = mn;
       float psum = 0.f;
       uint2 pk[2];
@@ -230,7 +236,7 @@ qsa_gqa_rows_mfma(const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc,
         float p[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          p[r] = s4[pt][r] > NEG_BIG ? exp2f(s4[pt][r] - mn) : 0.f;
+          p[r] = exp2_hw(s4[pt][r] - mn);
           psum += p[r];
         }
         pk[pt] = make_uint2(cvt_bf16x2(p[0], p[1]), cvt_bf16x2(p[2], p[3]));
@@ -264,49 +270,77 @@ qsa_gqa_rows_mfma(const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc,
 }
 
 // Splits -> normalized, gated output; the sink joins the denominator here.
-// A wave merges one (row, head); statistics are in powers of two.
+// Statistics are in powers of two.  WPR waves merge one (row, head): one where
+// there are few splits, four that share them otherwise.
+template <int WPR>
 __global__ void __launch_bounds__(256)
 qsa_gqa_merge(const float* __restrict__ part_o,
               const float* __restrict__ part_ml,
               const float* __restrict__ sink, const bf16_t* __restrict__ gate,
               long long gstride, bf16_t* __restrict__ out, long long ostride,
               long long total, int H, int E, int NS, float out_scale) {
-  const long long rh = (long long)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (rh >= total) return;
+  __shared__ float2 red[WPR == 1 ? 1 : WPR][64];
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int sub = wave % WPR;
+  const long long rh = (long long)blockIdx.x * (4 / WPR) + wave / WPR;
+  if (rh >= total) return;                        // WPR 4: never
   const int h = (int)(rh % H), lane = threadIdx.x & 63;
   const long long row = rh / H;
-  const float* ml = part_ml + rh * NS * 2;
+  const float2* ml = reinterpret_cast<const float2*>(part_ml) + rh * NS;
   const float sk = sink ? sink[h] * LOG2E : NEG_BIG;
   float top = NEG_BIG;
   for (int s = lane; s < NS; s += 64)
-    if (ml[2 * s + 1] > 0.f) top = fmaxf(top, ml[2 * s]);
+    if (ml[s].y > 0.f) top = fmaxf(top, ml[s].x);
   top = fmaxf(wave_reduce_max(top), sk);
   float den = 0.f;
   for (int s = lane; s < NS; s += 64)
-    if (ml[2 * s + 1] > 0.f)
-      den = fmaf(exp2f(ml[2 * s] - top), ml[2 * s + 1], den);
-  den = wave_reduce_sum(den) + (sink ? exp2f(sk - top) : 0.f);
+    if (ml[s].y > 0.f) den = fmaf(exp2_hw(ml[s].x - top), ml[s].y, den);
+  den = wave_reduce_sum(den) + (sink ? exp2_hw(sk - top) : 0.f);
   const float inv = den > 0.f ? out_scale / den : 0.f;
-  for (int e = lane * 2; e < E; e += 128) {       // E % 8 == 0
+  for (int e0 = 0; e0 < E; e0 += 128) {           // E % 8 == 0
+    const int e = e0 + lane * 2;
+    const bool in = e < E;
+    const float* po = part_o + rh * NS * E + (in ? e : 0);
     float a0 = 0.f, a1 = 0.f;
-    const float* po = part_o + rh * NS * E + e;
+    for (int s0 = 0; s0 < NS; s0 += 64) {
+      const int n = min(64, NS - s0);
+      float w = 0.f;
+      if (lane < n && ml[s0 + lane].y > 0.f)
+        w = exp2_hw(ml[s0 + lane].x - top);
 #pragma unroll 8
-    for (int s = 0; s < NS; ++s) {
-      const float w = ml[2 * s + 1] > 0.f ? exp2f(ml[2 * s] - top) : 0.f;
-      const float2 v = *reinterpret_cast<const float2*>(po + (long long)s * E);
-      a0 = fmaf(w, v.x, a0);
-      a1 = fmaf(w, v.y, a1);
+      for (int s = sub; s < n; s += WPR) {
+        const float ws = __shfl(w, s, QSA_WAVE);
+        const float2 v = *reinterpret_cast<const float2*>(
+            po + (long long)(s0 + s) * E);
+        a0 = fmaf(ws, v.x, a0);
+        a1 = fmaf(ws, v.y, a1);
+      }
     }
-    a0 *= inv;
-    a1 *= inv;
-    if (gate) {
-      const float2 gv = bf16x2_to_f32x2(*reinterpret_cast<const unsigned int*>(
-          gate + row * gstride + (long long)h * E + e));
-      a0 /= 1.f + __expf(-gv.x);
-      a1 /= 1.f + __expf(-gv.y);
+    if (WPR > 1) {
+      red[sub % WPR][lane] = make_float2(a0, a1);
+      __syncthreads();
+      if (sub == 0) {
+#pragma unroll
+        for (int k = 1; k < WPR; ++k) {
+          a0 += red[k][lane].x;
+          a1 += red[k][lane].y;
+        }
+      }
+      __syncthreads();
     }
-    *reinterpret_cast<unsigned int*>(out + row * ostride + (long long)h * E +
-                                     e) = cvt_bf16x2(a0, a1);
+    if (sub == 0 && in) {
+      a0 *= inv;
+      a1 *= inv;
+      if (gate) {
+        const float2 gv = bf16x2_to_f32x2(
+            *reinterpret_cast<const unsigned int*>(
+                gate + row * gstride + (long long)h * E + e));
+        a0 /= 1.f + __expf(-gv.x);
+        a1 /= 1.f + __expf(-gv.y);
+      }
+      *reinterpret_cast<unsigned int*>(out + row * ostride + (long long)h * E +
+                                       e) = cvt_bf16x2(a0, a1);
+    }
   }
 }
 
@@ -336,9 +370,14 @@ extern "C" void qsa_gqa_rows_mfma_launch(
 #undef QSA_GM_E
 #undef QSA_GM
   const long long total = (long long)R * H;
-  hipLaunchKernelGGL(qsa_gqa_merge, dim3((unsigned)((total + 3) / 4)),
-                     dim3(256), 0, st, part_o, part_ml, sink, gate, gstride,
-                     out, ostride, total, H, E, NS, out_scale);
+  if (NS > 8)
+    hipLaunchKernelGGL((qsa_gqa_merge<4>), dim3((unsigned)total), dim3(256),
+                       0, st, part_o, part_ml, sink, gate, gstride, out,
+                       ostride, total, H, E, NS, out_scale);
+  else
+    hipLaunchKernelGGL((qsa_gqa_merge<1>), dim3((unsigned)((total + 3) / 4)),
+                       dim3(256), 0, st, part_o, part_ml, sink, gate, gstride,
+                       out, ostride, total, H, E, NS, out_scale);
 }
 
 // ---------------------------------------------------------------------------
@@ -478,7 +517,8 @@ qsa_gqa_portions(const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc,
       mx = fmaxf(mx, __shfl_xor(mx, 16, QSA_WAVE));
       mx = fmaxf(mx, __shfl_xor(mx, 32, QSA_WAVE));
       const float mn = fmaxf(m[u], mx);
-      const float alpha = m[u] > NEG_BIG ? exp2f(m[u] - mn) : 0.f;
+      const float alpha = exp2_hw(m[u] - mn);     // page 0 shows every row a
+                                                  // key: mn is finite
       m[u] = mn;
       float psum = 0.f;
       uint2 pk[4];
@@ -487,7 +527,7 @@ qsa_gqa_portions(const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc,
         float p[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          p[r] = s4[u][pt][r] > NEG_BIG ? exp2f(s4[u][pt][r] - mn) : 0.f;
+          p[r] = exp2_hw(s4[u][pt][r] - mn);
           psum += p[r];
         }
         pk[pt] = make_uint2(cvt_bf16x2(p[0], p[1]), cvt_bf16x2(p[2], p[3]));

@@ -48,11 +48,12 @@ __device__ __forceinline__ ConvSpan conv_span(const ConvStep& st, int c) {
   return s;
 }
 
-// NP (1 or 2) groups of VEC channels, c0.. and c1..; TAPS 0: `taps` of them, through memory.
-template <typename T, int TAPS, int VEC, int NP, typename Emit>
+// NP (1 or 2) groups of VEC channels, c0.. and c1..; TAPS 0: `taps` of them,
+// through memory.  pre(t) loads what emit(t, values, .) wants besides.
+template <typename T, int TAPS, int VEC, int NP, typename Pre, typename Emit>
 __device__ __forceinline__ void conv_rows(
     const T* x, long long xstride, T* tail, int C, int c0, int c1,
-    const float* w, const float* bias, int taps, const ConvSpan& s,
+    const float* w, const float* bias, int taps, const ConvSpan& s, Pre pre,
     Emit emit) {
   const int NT = (TAPS ? TAPS : taps) - 1;
   auto ch = [&](int p) { return p == 0 ? c0 : c1; };
@@ -90,6 +91,7 @@ __device__ __forceinline__ void conv_rows(
     }
 #pragma unroll 4
     for (int t = s.t0; t < s.t1; ++t) {
+      const auto aux = pre(t);
       float a[NP][VEC];
 #pragma unroll
       for (int p = 0; p < NP; ++p) {
@@ -107,10 +109,11 @@ __device__ __forceinline__ void conv_rows(
           win[p][K - 1][i] = u[i];
         }
       }
-      emit(t, a);
+      emit(t, a, aux);
     }
   } else {
     for (int t = s.t0; t < s.t1; ++t) {
+      const auto aux = pre(t);
       float a[NP][VEC];
 #pragma unroll
       for (int p = 0; p < NP; ++p) {
@@ -124,7 +127,7 @@ __device__ __forceinline__ void conv_rows(
           for (int i = 0; i < VEC; ++i) a[p][i] = fmaf(wj[i], u[i], a[p][i]);
         }
       }
-      emit(t, a);
+      emit(t, a, aux);
     }
   }
   if (s.t0 == 0) {
@@ -139,17 +142,23 @@ __device__ __forceinline__ void conv_rows(
   }
 }
 
-#define CONV_CASE(T, TAPS, VEC, NP, emit)                                    \
+#define CONV_CASE(T, TAPS, VEC, NP)                                          \
   conv_rows<T, TAPS, VEC, NP>(x, xstride, tail, C, c0, c1, w, bias, taps, s, \
-                              emit)
-#define CONV_DISPATCH(T, VEC, NP, emit)              \
-  switch (taps) {                                    \
-    case 1: CONV_CASE(T, 1, VEC, NP, emit); break;   \
-    case 2: CONV_CASE(T, 2, VEC, NP, emit); break;   \
-    case 3: CONV_CASE(T, 3, VEC, NP, emit); break;   \
-    case 4: CONV_CASE(T, 4, VEC, NP, emit); break;   \
-    default: CONV_CASE(T, 0, VEC, NP, emit);         \
+                              pre, emit)
+#define CONV_DISPATCH(T, VEC, NP)              \
+  switch (taps) {                              \
+    case 1: CONV_CASE(T, 1, VEC, NP); break;   \
+    case 2: CONV_CASE(T, 2, VEC, NP); break;   \
+    case 3: CONV_CASE(T, 3, VEC, NP); break;   \
+    case 4: CONV_CASE(T, 4, VEC, NP); break;   \
+    default: CONV_CASE(T, 0, VEC, NP);         \
   }
+
+template <int VEC>
+struct Turn {
+  int slot;                    // where k or v goes
+  float c[VEC], s[VEC];
+};
 
 // A thread owns a pair of channel groups: of q and k a rotated pair (i,
 // i + rot/2) or two groups behind the rotated ones, of v two groups.
@@ -183,35 +192,42 @@ qsa_conv_qkv(const T* x, long long xstride, const float* __restrict__ w,
   const int d1 = two ? far : d0;
   const int base = val ? (H + G) * D + head * E : head * D;
   const int c0 = base + d0, c1 = base + d1;
-  auto emit = [=](int t, float (&a)[2][VEC]) {
+  const bool query = !val && head < H;
+  auto pre = [=](int t) {
+    Turn<VEC> r;
+    r.slot = query ? 0 : cache_slots[s.r0 + t];
+    if (turn) {
+      const long long at =
+          (long long)min(s.p0 + t, table_len - 1) * half + d0;
+      ldv<float, VEC>(cos_t + at, r.c);
+      ldv<float, VEC>(sin_t + at, r.s);
+    }
+    return r;
+  };
+  auto emit = [=](int t, float (&a)[2][VEC], const Turn<VEC>& r) {
     const long long row = s.r0 + t;
     if (turn) {
-      const int p = min(s.p0 + t, table_len - 1);
-      float cc[VEC], ss[VEC];
-      ldv<float, VEC>(cos_t + (long long)p * half + d0, cc);
-      ldv<float, VEC>(sin_t + (long long)p * half + d0, ss);
 #pragma unroll
       for (int i = 0; i < VEC; ++i) {
         const float u0 = a[0][i], v0 = a[1][i];
-        a[0][i] = u0 * cc[i] - v0 * ss[i];
-        a[1][i] = v0 * cc[i] + u0 * ss[i];
+        a[0][i] = u0 * r.c[i] - v0 * r.s[i];
+        a[1][i] = v0 * r.c[i] + u0 * r.s[i];
       }
     }
     T* dst;
-    if (!val && head < H) {
+    if (query) {
       dst = q + (row * H + head) * D;
     } else {
-      const int slot = cache_slots[row];
-      if (slot < 0) return;
-      const long long at = (long long)(slot >> 6) * G +
+      if (r.slot < 0) return;
+      const long long at = (long long)(r.slot >> 6) * G +
                            (val ? head : head - H);
-      dst = val ? vc + (at * 64 + (slot & 63)) * E
-                : kc + (at * 64 + (slot & 63)) * D;
+      dst = val ? vc + (at * 64 + (r.slot & 63)) * E
+                : kc + (at * 64 + (r.slot & 63)) * D;
     }
     stv<T, VEC>(dst + d0, a[0]);
     if (two) stv<T, VEC>(dst + d1, a[1]);
   };
-  CONV_DISPATCH(T, VEC, 2, emit)
+  CONV_DISPATCH(T, VEC, 2)
 }
 
 extern "C" void qsa_conv_qkv_launch(
@@ -245,14 +261,15 @@ qsa_conv_silu(const T* x, long long xstride, const float* __restrict__ w,
   if (s.slot < 0 || s.p0 < 0) return;
   T* tail = tails + (long long)s.slot * (taps - 1) * C;
   const int c0 = u * VEC, c1 = c0;
-  auto emit = [=](int t, float (&a)[1][VEC]) {
+  auto pre = [](int) { return 0; };
+  auto emit = [=](int t, float (&a)[1][VEC], int) {
 #pragma unroll
     for (int i = 0; i < VEC; ++i)
       a[0][i] = sizeof(T) == 4 ? silu_f(a[0][i])
                                : a[0][i] / (1.f + __expf(-a[0][i]));
     stv<T, VEC>(out + (long long)(s.r0 + t) * C + c0, a[0]);
   };
-  CONV_DISPATCH(T, VEC, 1, emit)
+  CONV_DISPATCH(T, VEC, 1)
 }
 
 extern "C" void qsa_conv_silu_launch(const void* x, long long xstride,

@@ -44,7 +44,8 @@ def test_mixer_kernels(lm_stats):
     """Matrix kernels issue MFMA, nothing spills vector registers or uses
     scratch, and no packed f32 arithmetic was formed."""
     for frag in ("retention_state", "retention_out", "latent_rows_mfma",
-                 "window_attn_prefill", "head_matmul_mfma", "skinny_gemm"):
+                 "window_attn_prefill", "head_matmul_mfma", "skinny_gemm",
+                 "gqa_rows_mfma", "gqa_portions", "ssd_state", "ssd_out"):
         for name, st in _named(lm_stats, frag).items():
             assert st["mfma"] >= 4, f"{name}: only {st['mfma']} v_mfma"
     for name, st in lm_stats.items():
