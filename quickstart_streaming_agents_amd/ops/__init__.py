@@ -1,8 +1,9 @@
 """Op layer: the hand-written HIP/CDNA4 kernels + CPU references.
 
 Two native modules: qsa_hip (streaming, retrieval, Llama/Mixtral/encoder
-kernels) and qsa_lm_hip (mixer decoders: retention, latent attention, f32
-residual norms, greedy pick).
+kernels) and qsa_lm_hip (mixer decoders: retention, latent and grouped-query
+attention, short convolutions, state-space duality, f32 residual norms, greedy
+pick).
 
 Fail-loud contract: on a GPU box the HIP extension MUST be importable —
 there is no silent eager fallback for the hot ops.  CPU-only environments
